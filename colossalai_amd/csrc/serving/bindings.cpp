@@ -27,7 +27,7 @@ at::Tensor paged_attention_ext(at::Tensor q, at::Tensor kpool, at::Tensor vpool,
                                double softcap, bool sink, c10::optional<at::Tensor> sink_logits,
                                c10::optional<at::Tensor> dist_bias, c10::optional<at::Tensor> ksum,
                                c10::optional<at::Tensor> vsum, int64_t sum_block, bool cross, int64_t num_tiles,
-                               int64_t num_tiles128);
+                               int64_t num_tiles128, int64_t chunk, c10::optional<at::Tensor> key_fac, bool out_f32);
 void paged_pool_write(at::Tensor kpool, at::Tensor vpool, at::Tensor ksum, at::Tensor vsum, at::Tensor block_tables,
                       at::Tensor cu, at::Tensor start, int64_t block, int64_t most_blocks);
 at::Tensor rotate_halves_unit_norm(at::Tensor x, at::Tensor positions, c10::optional<at::Tensor> freqs, double eps,
@@ -49,6 +49,15 @@ at::Tensor expert_combine(at::Tensor y, at::Tensor inv, at::Tensor weights, c10:
                           c10::optional<at::Tensor> base_gate, c10::optional<at::Tensor> ids, int64_t num_experts,
                           c10::optional<at::Tensor> identity_rows);
 at::Tensor gelu_tanh_mul(at::Tensor packed);
+at::Tensor relu_mul(at::Tensor packed);
+at::Tensor query_norm_key_write(at::Tensor q, at::Tensor k, at::Tensor weight, double eps, double coef, double every,
+                                at::Tensor positions, at::Tensor kpool, at::Tensor kfac, at::Tensor rows);
+at::Tensor difference_norm(at::Tensor o, int64_t kv_heads, double lam, double mult, double eps, at::ScalarType out_dtype);
+std::vector<at::Tensor> streams_start(at::Tensor table, at::Tensor tokens, int64_t streams, at::Tensor w_in,
+                                      at::Tensor weight, double eps);
+c10::optional<at::Tensor> streams_update(at::Tensor x, at::Tensor y, at::Tensor mix, at::Tensor w_out,
+                                         c10::optional<at::Tensor> w_in, c10::optional<at::Tensor> weight, double eps,
+                                         at::ScalarType out_dtype);
 at::Tensor gated_grouped_rms_norm(at::Tensor x, at::Tensor gate, at::Tensor weight, int64_t groups, double eps,
                                   at::ScalarType out_dtype);
 c10::optional<at::Tensor> add_layer_norm(c10::optional<at::Tensor> residual, at::Tensor y,
@@ -75,7 +84,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("merge_rms_norm", &s::merge_rms_norm, "average of two RMS-normed branches, group norm, residual add");
   m.def("paged_attention", &s::paged_attention, "ragged paged attention: window, kept prefix, distance bias, gate, soft cap, sink");
   m.def("paged_attention_ext", &s::paged_attention_ext,
-        "split-key ragged paged attention with a learned sink, a distance table, block summaries, cross-head values");
+        "ragged paged attention with a learned sink, a distance table, block summaries, cross-head values, fixed blocks "
+        "of positions, key factors, shared value heads, float32 output");
   m.def("paged_pool_write", &s::paged_pool_write, "means of the key/value blocks a step completes, into the summary pools");
   m.def("rotate_halves_unit_norm", &s::rotate_halves_unit_norm, "rotate-half rotary on the first channels, then unit RMS per head");
   m.def("lerp_rows", &s::lerp_rows, "(1 - lam) a + lam b, float32 inside");
@@ -87,6 +97,12 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("grouped_topk_route", &s::grouped_topk_route,
         "sigmoid or softmax router: correction, group-limited top-k, renormalised or not");
   m.def("gelu_tanh_mul", &s::gelu_tanh_mul, "gelu_tanh(gate) * up of a packed [N, 2F] tensor");
+  m.def("relu_mul", &s::relu_mul, "max(gate, 0) * up of a packed [N, 2F] tensor");
+  m.def("query_norm_key_write", &s::query_norm_key_write,
+        "RMS norm + position growth of queries; raw keys and their 1 / rms into the pool");
+  m.def("difference_norm", &s::difference_norm, "unit RMS of the difference of two attention maps' outputs, scaled");
+  m.def("streams_start", &s::streams_start, "embedding rows as parallel residual streams, and the first sublayer's input");
+  m.def("streams_update", &s::streams_update, "write a sublayer's output into the streams, read and norm the next input");
   m.def("gated_grouped_rms_norm", &s::gated_grouped_rms_norm, "x * silu(gate), then grouped RMS norm");
   m.def("add_layer_norm", &s::add_layer_norm,
         "residual += mult * layer_norm(y) * w_out in place, then the layer norm of the sum (weight, no bias)");

@@ -1,7 +1,8 @@
 // Element-wise serving kernels: token shift with carried previous row,
-// squared ReLU, gated SiLU / tanh-GELU of a packed tensor, logit soft-cap, ragged
-// scatter of keys/values into pages, rotary positions on neighbouring pairs, and
-// the write of a latent-attention row (norm + rotation + scatter).
+// squared ReLU, gated SiLU / tanh-GELU / ReLU of a packed tensor, logit soft-cap, ragged
+// scatter of keys/values into pages, rotary positions on neighbouring pairs, the
+// write of a latent-attention row (norm + rotation + scatter), and the query norm +
+// raw key write of attention whose values are its keys.
 #include "serving_common.h"
 
 namespace cai {
@@ -136,12 +137,14 @@ void paged_kv_write(at::Tensor k, at::Tensor v, at::Tensor kpool, at::Tensor vpo
   HIP_CHECK_LAST();
 }
 
-// packed [N, 2F] = [gate | up], rows strided by ps -> out [N, F] = silu(gate) * up, formed in float32.
+// packed [N, 2F] = [gate | up], rows strided by ps -> out [N, F] = act(gate) * up, formed in float32.
 // VEC: eight elements per thread (F and the row stride are multiples of 8 and the base is aligned).
-// ACT: 0 = silu(g) = g * sigmoid(g); 1 = the tanh form of GELU, 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))).
+// ACT: 0 = silu(g) = g * sigmoid(g); 1 = the tanh form of GELU, 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3)));
+// 2 = ReLU, max(g, 0).
 template <int ACT>
 DEV_INLINE float gate_act(float g) {
   if (ACT == 0) return g * sigmoidf_(g);
+  if (ACT == 2) return fmaxf(g, 0.0f);
   return 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
 }
 
@@ -190,6 +193,7 @@ static at::Tensor gated_act_mul(at::Tensor packed) {
 
 at::Tensor silu_mul(at::Tensor packed) { return gated_act_mul<0>(packed); }
 at::Tensor gelu_tanh_mul(at::Tensor packed) { return gated_act_mul<1>(packed); }
+at::Tensor relu_mul(at::Tensor packed) { return gated_act_mul<2>(packed); }
 
 // ------------------------------------------------------------ rotary on pairs
 // The pair (2i, 2i + 1), i < half, of a vector at position p turns by a = p * freqs[i], float32.
@@ -394,6 +398,88 @@ at::Tensor rotate_halves_unit_norm(at::Tensor x, at::Tensor positions, c10::opti
     });
   });
 #undef RH_LAUNCH
+  HIP_CHECK_LAST();
+  return out;
+}
+
+// --------------------------------------------- query norm, raw key write
+// Attention whose keys are normed but whose values are the raw keys caches one row per token and kv head: the key as
+// projected, and the float32 factor 1 / rms that turns it into a normed key when it is read. One wave per (token, head of
+// the H query + G key heads). Query: out = q * w / sqrt(mean(q^2) + eps) * (1 + coef ln(floor((p + 1) / every) + 1))
+// (every = 0: no growth with position; w holds the query norm's weight times the key norm's). Key: the row goes to
+// pool row rows[n] as it is, 1 / sqrt(mean(k^2) + eps) to its factor. The row stays in registers (D <= 64 * PER).
+template <typename T, int PER>
+__global__ __launch_bounds__(256) void query_norm_key_write_kernel(
+    T* __restrict__ out, T* __restrict__ kpool, float* __restrict__ kfac, const T* __restrict__ q, long qs,
+    const T* __restrict__ k, long ks, const float* __restrict__ w, const int* __restrict__ positions,
+    const int* __restrict__ rows, long units, int H, int G, int D, float eps, float coef, double every) {
+  const int lane = threadIdx.x & 63;
+  const long unit = (long)blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
+  if (unit >= units) return;
+  const long n = unit / (H + G);
+  const int hd = (int)(unit % (H + G));
+  const bool query = hd < H;
+  const T* src = query ? q + n * qs + (long)hd * D : k + n * ks + (long)(hd - H) * D;
+  float v[PER], ssq = 0.0f;
+#pragma unroll
+  for (int r = 0; r < PER; ++r) {
+    const int d = lane + 64 * r;
+    v[r] = d < D ? ldf(src + d) : 0.0f;
+    ssq += v[r] * v[r];
+  }
+  const float inv = 1.0f / sqrtf(wave_reduce_sum(ssq) / (float)D + eps);
+  if (query) {
+    float f = inv;
+    if (every > 0.0) f *= 1.0f + coef * logf((float)(floor((double)(positions[n] + 1) / every) + 1.0));
+#pragma unroll
+    for (int r = 0; r < PER; ++r) {
+      const int d = lane + 64 * r;
+      if (d < D) stf(out + (n * H + hd) * (long)D + d, v[r] * f * w[d]);
+    }
+  } else {
+    const long row = (long)rows[n] * G + (hd - H);
+#pragma unroll
+    for (int r = 0; r < PER; ++r) {
+      const int d = lane + 64 * r;
+      if (d < D) stf(kpool + row * D + d, v[r]);
+    }
+    if (lane == 0) kfac[row] = inv;
+  }
+}
+
+at::Tensor query_norm_key_write(at::Tensor q, at::Tensor k, at::Tensor weight, double eps, double coef, double every,
+                                at::Tensor positions, at::Tensor kpool, at::Tensor kfac, at::Tensor rows) {
+  check_act(q, "q"); check_act(k, "k");
+  TORCH_CHECK(q.dim() == 3 && k.dim() == 3 && q.size(0) == k.size(0) && q.size(2) == k.size(2) &&
+              q.scalar_type() == k.scalar_type(), "q must be [N, H, D], k [N, G, D] of one type");
+  const long N = q.size(0);
+  const int H = (int)q.size(1), G = (int)k.size(1), D = (int)q.size(2);
+  TORCH_CHECK(q.stride(2) == 1 && (H == 1 || q.stride(1) == D) && k.stride(2) == 1 && (G == 1 || k.stride(1) == D),
+              "the heads of a token must lie side by side");
+  TORCH_CHECK(D <= 512, "head sizes up to 512");
+  TORCH_CHECK(kpool.is_cuda() && kpool.is_contiguous() && kpool.dim() == 4 && kpool.size(2) == G && kpool.size(3) == D &&
+              kpool.scalar_type() == q.scalar_type(), "pool must be contiguous [pages, page, G, D] of q's type");
+  TORCH_CHECK(kfac.is_cuda() && is_f32(kfac) && kfac.is_contiguous() && kfac.dim() == 3 && kfac.size(0) == kpool.size(0) &&
+              kfac.size(1) == kpool.size(1) && kfac.size(2) == G, "key factors must be contiguous float32 [pages, page, G]");
+  check_i32(positions, "positions"); check_i32(rows, "rows");
+  at::Tensor w = f32c(weight);
+  TORCH_CHECK(w.is_cuda() && w.numel() == D && positions.numel() == N && rows.numel() == N && every >= 0.0);
+  at::Tensor out = at::empty({N, H, D}, q.options());
+  const long units = N * (H + G);
+  if (units == 0) return out;
+  const dim3 grid((unsigned)((units + 3) / 4));
+#define QNK_LAUNCH(PER_)                                                                                            \
+  hipLaunchKernelGGL((query_norm_key_write_kernel<T, PER_>), grid, dim3(256), 0, stream(), ptr<T>(out), ptr<T>(kpool), \
+                     kfac.data_ptr<float>(), ptr<T>(q), (long)q.stride(0), ptr<T>(k), (long)k.stride(0),             \
+                     w.data_ptr<float>(), positions.data_ptr<int>(), rows.data_ptr<int>(), units, H, G, D,           \
+                     (float)eps, (float)coef, every)
+  SERVING_DISPATCH_ACT(q, T, {
+    if (D <= 64) QNK_LAUNCH(1);
+    else if (D <= 128) QNK_LAUNCH(2);
+    else if (D <= 256) QNK_LAUNCH(4);
+    else QNK_LAUNCH(8);
+  });
+#undef QNK_LAUNCH
   HIP_CHECK_LAST();
   return out;
 }

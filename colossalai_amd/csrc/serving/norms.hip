@@ -13,7 +13,9 @@
 //   add_layer_norm     : centred norm (weight, no bias) of a sublayer's output
 //                        added, scaled, to the residual in place, and the
 //                        centred norm of the new residual row for the next
-//                        sublayer, in one launch.
+//                        sublayer, in one launch;
+//   difference_norm    : a1 - lambda a2 of two attention maps' outputs per head,
+//                        unit RMS over the head, a constant factor.
 #include "serving_common.h"
 
 namespace cai {
@@ -642,6 +644,59 @@ c10::optional<at::Tensor> add_scaled_unit_norm(at::Tensor residual, at::Tensor a
     HIP_CHECK_LAST();
   }
   if (!out_dtype.has_value()) return c10::nullopt;
+  return out;
+}
+
+// ------------------------------------------------------- difference of two attention maps
+// o [N, G, 2, R, Dv] float32: the outputs of map 1 and map 2 of the R query heads of every kv head. One wave per
+// (token, head g * R + r): d = a1 - lam * a2, out = d / sqrt(mean(d^2) + eps) * mult, heads in order. d stays in
+// registers (Dv <= 64 * PER).
+template <typename TO, int PER>
+__global__ __launch_bounds__(256) void difference_norm_kernel(TO* __restrict__ out, const float* __restrict__ o, long units,
+                                                              int H, int R, int Dv, float lam, float mult, float eps) {
+  const int lane = threadIdx.x & 63;
+  const long unit = (long)blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
+  if (unit >= units) return;
+  const long n = unit / H;
+  const int h = (int)(unit % H), g = h / R, r = h % R;
+  const float* a1 = o + (n * 2 * H + (long)(2 * g) * R + r) * Dv;
+  const float* a2 = a1 + (long)R * Dv;
+  float d[PER], ssq = 0.0f;
+#pragma unroll
+  for (int p = 0; p < PER; ++p) {
+    const int i = lane + 64 * p;
+    d[p] = i < Dv ? a1[i] - lam * a2[i] : 0.0f;
+    ssq += d[p] * d[p];
+  }
+  const float f = mult / sqrtf(wave_reduce_sum(ssq) / (float)Dv + eps);
+#pragma unroll
+  for (int p = 0; p < PER; ++p) {
+    const int i = lane + 64 * p;
+    if (i < Dv) stf(out + unit * Dv + i, d[p] * f);
+  }
+}
+
+at::Tensor difference_norm(at::Tensor o, int64_t kv_heads, double lam, double mult, double eps, at::ScalarType out_dtype) {
+  TORCH_CHECK(o.is_cuda() && is_f32(o) && o.dim() == 3 && o.is_contiguous(), "o must be contiguous float32 [N, 2H, Dv]");
+  const long N = o.size(0);
+  const int H = (int)(o.size(1) / 2), Dv = (int)o.size(2);
+  TORCH_CHECK(o.size(1) == 2 * H && kv_heads > 0 && H % kv_heads == 0 && Dv <= 512, "heads must split over the kv heads");
+  TORCH_CHECK(out_dtype == at::kFloat || out_dtype == at::kBFloat16);
+  at::Tensor out = at::empty({N, (long)H * Dv}, o.options().dtype(out_dtype));
+  const long units = N * H;
+  if (units == 0) return out;
+  const dim3 grid((unsigned)((units + 3) / 4));
+#define DN_LAUNCH(PER_)                                                                                        \
+  hipLaunchKernelGGL((difference_norm_kernel<TO, PER_>), grid, dim3(256), 0, stream(), ptr<TO>(out),           \
+                     o.data_ptr<float>(), units, H, (int)(H / kv_heads), Dv, (float)lam, (float)mult, (float)eps)
+  SERVING_DISPATCH_ACT(out, TO, {
+    if (Dv <= 64) DN_LAUNCH(1);
+    else if (Dv <= 128) DN_LAUNCH(2);
+    else if (Dv <= 256) DN_LAUNCH(4);
+    else DN_LAUNCH(8);
+  });
+#undef DN_LAUNCH
+  HIP_CHECK_LAST();
   return out;
 }
 

@@ -3,8 +3,10 @@
 // soft cap on the scaled score and an optional sink (one more place of score 0
 // in the softmax denominator that carries no value; with sink logits its score is learned per
 // head), an additive per-distance table, block summaries (one mean key/value per block of
-// positions that lies wholly before the window, kept in a small pool of their own) and, for
-// talking heads, every query head's weights applied to every key/value head's values.
+// positions that lies wholly before the window, kept in a small pool of their own; for
+// talking heads, every query head's weights applied to every key/value head's values), visibility
+// inside fixed blocks of positions instead of a window, a float32 factor per cached key (keys that
+// are normed when they are read), value heads shared by several key heads, and float32 output.
 //
 // One wave per (token, query head). The visible keys of a token are two
 // position ranges: the kept prefix [0, min(keep_first, lo)) and the window
@@ -32,6 +34,12 @@ DEV_INLINE float dpp_add(float v) {
 // sum over the 8 adjacent lanes that share a key (quad xor 1, quad xor 2, half-row mirror)
 DEV_INLINE float reduce8(float v) { return dpp_add<0x141>(dpp_add<0x4E>(dpp_add<0xB1>(v))); }
 
+// First position a query at `pos` sees: its block of `chunk` positions, its window, or position 0.
+DEV_INLINE int first_visible(int pos, int window, int chunk) {
+  if (chunk > 0) return pos - pos % chunk;
+  return window > 0 ? max(0, pos - window + 1) : 0;
+}
+
 // Scalar kernel (decode tokens, float32 serving, shapes the MFMA kernel does not take).
 // One block per (token, kv head, group of up to RC query heads of that kv head): keys and
 // values are read once for the whole group. The block's nw waves (16, or 8 when the partial
@@ -55,12 +63,15 @@ __global__ __launch_bounds__(64 * ATT_WAVES) void paged_attention_kernel(
     int H, int G, int D, int Dv, int page_shift, float scale, int window, int keep_first, int kvec, int vvec,
     float softcap, int sink, long vrow, long vhead, const float* __restrict__ sink_logits,
     const float* __restrict__ dist_bias, int dist_rows, const T* __restrict__ ksum, const T* __restrict__ vsum,
-    int sum_shift, int sum_block, float* __restrict__ cross_out) {
+    int sum_shift, int sum_block, float* __restrict__ cross_out, int chunk, const float* __restrict__ key_fac, int vrep,
+    float* __restrict__ out32) {
   // sink_logits [H]: the sink's score per head instead of 0. dist_bias [dist_rows, H]: added to the score of a key at
   // distance d (row min(d, dist_rows - 1)). ksum / vsum: block summaries, rows [pages << sum_shift]; a query at
   // `pos` sees the first max(0, (pos - window + 1) / sum_block) of its sequence's, ahead of its other keys and
   // without distance terms. cross_out [N, H, G, Dv] float32: the grid then has G blocks per (token, kv head, chunk),
-  // block c applies the heads' weights to the values of kv head c.
+  // block c applies the heads' weights to the values of kv head c. chunk > 0: a query sees its own block of `chunk`
+  // positions only (counted from position 0). key_fac [pool rows, G]: the cached key's score is multiplied by it. vrep:
+  // key heads per value head (the value pool has G / vrep heads). out32 [N, H, Dv]: float32 output instead of `out`.
   // vrow / vhead: elements between the value rows of neighbouring pool rows / kv heads (G * Dv and Dv for a
   // pool of its own; a value pool that is a view into wider rows, e.g. the leading channels of the keys, has others)
   extern __shared__ __align__(16) float lds[];
@@ -75,7 +86,7 @@ __global__ __launch_bounds__(64 * ATT_WAVES) void paged_attention_kernel(
   const long bx = blockIdx.x / VC;
   const long n = bx / (G * chunks);
   const int g = (int)(bx / chunks) % G;
-  const int vg = cross_out != nullptr ? (int)(blockIdx.x % VC) : g;  // kv head whose values this block reads
+  const int vg = cross_out != nullptr ? (int)(blockIdx.x % VC) : g / vrep;  // kv head whose values this block reads
   const int h0 = g * R + (int)(bx % chunks) * RC;  // first query head of this block
   const int nh = min(RC, g * R + R - h0);
   const int b = tok_seq[n];
@@ -92,7 +103,7 @@ __global__ __launch_bounds__(64 * ATT_WAVES) void paged_attention_kernel(
 #pragma unroll
   for (int r = 0; r < RC; ++r) slope[r] = (slopes != nullptr && r < nh) ? slopes[h0 + r] : 0.0f;
 
-  const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+  const int lo = first_visible(pos, window, chunk);
   const int n_sum = (ksum != nullptr && window > 0) ? max(0, (pos - window + 1) / sum_block) : 0;
   const int sum_mask = (1 << sum_shift) - 1;
   const int n_keep = (window > 0 ? min(keep_first, lo) : 0) + n_sum;  // summaries, then kept first tokens
@@ -156,6 +167,7 @@ __global__ __launch_bounds__(64 * ATT_WAVES) void paged_attention_kernel(
 #pragma unroll
         for (int r = 0; r < RC; ++r) {
           float sc = dots[r] * scale;
+          if (key_fac != nullptr && !summary) sc *= key_fac[(long)row * G + g];
           if (softcap > 0.0f) sc = softcap * tanhf(sc * inv_cap);
           if (!summary) {
             sc -= slope[r] * (float)(pos - j);
@@ -277,6 +289,7 @@ __global__ __launch_bounds__(64 * ATT_WAVES) void paged_attention_kernel(
     float scale_out = 1.0f / ll;
     if (gate != nullptr) scale_out *= sigmoidf_(ldf(gate + n * gate_stride + h0 + r));
     if (cross_out != nullptr) cross_out[((n * H + h0 + r) * G + vg) * (long)Dv + dv] = o * scale_out;
+    else if (out32 != nullptr) out32[(n * H + h0 + r) * (long)Dv + dv] = o * scale_out;
     else stf(out + (n * H + h0 + r) * (long)Dv + dv, o * scale_out);
   }
 }
@@ -304,12 +317,13 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
     int H, int G, int Dr, int Dvr, int page_shift, float scale, int window, int keep_first, float softcap, int sink,
     int qsplit, const float* __restrict__ sink2, const float* __restrict__ dist2, int dist_rows,
     const bf16s* __restrict__ ksum, const bf16s* __restrict__ vsum, int sum_shift, int sum_block,
-    float* __restrict__ cross_out) {
+    float* __restrict__ cross_out, int chunk, const float* __restrict__ key_fac, int vrep, float* __restrict__ out32) {
   // The optional extras of the split-key kernel, in the base-2 domain: sink2 [H] = learned sink scores * log2e;
   // dist2 [H, dist_rows] = the per-distance bias * log2e, one row per head; ksum / vsum = block summaries, staged as
   // the first tiles of a block (summary idx of a sequence is seen by a token at pos when idx < (pos - window + 1) /
   // sum_block); cross_out [N, H, G, Dv] float32: the grid's z axis then also counts the kv head whose values a block
-  // multiplies the weights with.
+  // multiplies the weights with; chunk, key_fac [pool rows, G], vrep and out32 as in the split-key kernel (the factors of
+  // a key tile are staged with it).
   // qsplit (kv heads with a single query head each): the four waves of a block are four consecutive 32-token tiles
   // of that head instead of four heads, so a block covers 128 tokens, the grid's x axis counts 128-token tiles, and
   // the staged key/value tiles are still shared by all computing waves. The block stages the key range of all its
@@ -323,13 +337,15 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
   constexpr int KT = 32 * KP, VTT = Dv * VP;   // elements of one staged tile
   constexpr int KCH = 32 * D / 8, VCH = 32 * Dv / 8;  // 16-byte chunks of a key / value tile
   constexpr int TP = MFMA_TILES_PER_STEP;
-  extern __shared__ __align__(16) bf16s tiles[];  // [2][TP][KT + VTT]
+  extern __shared__ __align__(16) bf16s tiles[];  // [2][TP][KT + VTT], then [2][TP][32] key factors (float)
+  float* facs = reinterpret_cast<float*>(tiles + 2 * TP * (KT + VTT));
   constexpr int nthreads = 256;  // always four waves: those beyond the group's heads only help staging
   const int tid = threadIdx.x;
   const int wid = tid >> 6, lane = tid & 63;
   const int rep = H / G, g = blockIdx.y;
   const int VC = cross_out != nullptr ? G : 1;
-  const int vg = cross_out != nullptr ? (int)(blockIdx.z % VC) : g;   // kv head of the values
+  const int vg = cross_out != nullptr ? (int)(blockIdx.z % VC) : g / vrep;   // kv head of the values
+  const int Gv = G / vrep;
   const int hl = qsplit ? 0 : (blockIdx.z / VC) * (nthreads >> 6) + wid;  // head inside the group
   const int h = g * rep + (hl < rep ? hl : 0);
   const int bshift = qsplit ? 7 : 5;                  // log2 of the tokens a block covers
@@ -365,7 +381,9 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
   for (int s = 0; s < DS; ++s)
     qf[s] = 16 * s + hf * 8 < Dr ? ld_g16b(q + n * q_stride + (long)h * Dr + 16 * s + hf * 8) : zero8;
 
-  const int lo_min = window > 0 ? max(0, bp0 - window + 1) : 0;   // the staged key range is the block's
+  const int lo_min = first_visible(bp0, window, chunk);   // the staged key range is the block's
+  const int lo = first_visible(pos, window, chunk);       // this token's first key
+  const int lo_p0 = first_visible(p0, window, chunk), lo_p1 = first_visible(p1, window, chunk);  // the wave's
   const int wstart = lo_min & ~31;
   const int n_sink = window > 0 ? min(keep_first, wstart) : 0;  // kept keys below the window's first tile
   const int n_sum = (ksum != nullptr && window > 0) ? max(0, (bp1 - window + 1) / sum_block) : 0;  // the block's last token's
@@ -396,7 +414,8 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
   };
   // The page-table lookups of a tile run one tile ahead of its key/value loads (two ahead of its use), so that a
   // load's address never waits for a lookup issued in the same iteration.
-  int krow[TP][KR], vrow[TP][VR];
+  int krow[TP][KR], vrow[TP][VR], frow[TP];
+  float rf[TP];
   bool from_sum[TP];  // the tiles of the last lookup that are summary tiles
   auto lookup = [&](int step) {
 #pragma unroll
@@ -415,6 +434,7 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
         const int j = kbase + (c & 31);
         vrow[u][r] = c < VCH ? (int)(from_sum[u] ? sum_row(j) : pool_row(j)) : 0;
       }
+      if (key_fac != nullptr && tid < 32) frow[u] = (int)pool_row(kbase + tid);
     }
   };
   auto fetch = [&]() {  // the tiles whose rows the last lookup left in krow / vrow
@@ -435,9 +455,10 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
         const int c = tid + nthreads * r;
         if (c < VCH) {
           const int off = 8 * (c >> 5);
-          rv[u][r] = off < Dvr ? ld_g16b(vp + ((long)vrow[u][r] * G + vg) * Dvr + off) : zero8;
+          rv[u][r] = off < Dvr ? ld_g16b(vp + ((long)vrow[u][r] * Gv + vg) * Dvr + off) : zero8;
         }
       }
+      if (key_fac != nullptr && tid < 32) rf[u] = key_fac[(long)frow[u] * G + g];
     }
   };
   auto stash = [&](int buf) {
@@ -465,6 +486,7 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
           }
         }
       }
+      if (key_fac != nullptr && tid < 32) facs[(buf * TP + u) * 32 + tid] = rf[u];
     }
   };
 
@@ -513,7 +535,8 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
       const bool summ = it < sum_tiles;
       const bool sink = it < sink_tiles;  // a tile ahead of the window's: summaries or kept first tokens
       const int kbase = tile_base(it);
-      if (!sink && kbase > p1) continue;  // (query split) a tile wholly after this wave's tokens
+      // (query split) a tile wholly after this wave's tokens, or wholly before what they see
+      if (!sink && (kbase > p1 || (kbase + 31 < lo_p0 && kbase >= keep_first))) continue;
       const int klimit = sink ? n_sink : p1 + 1;  // keys of this tile at or above it are not this tile's to count
       const bf16s* ks = tiles + (buf * TP + u) * (KT + VTT);
       const bf16s* vt = ks + KT;
@@ -525,11 +548,20 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
         const bf16x8_v kf = *reinterpret_cast<const bf16x8_v*>(ks + col * KP + 16 * s + hf * 8);
         sacc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, qf[s], sacc, 0, 0, 0);
       }
+      if (key_fac != nullptr) {
+        const float* fc = facs + (buf * TP + u) * 32 + 4 * hf;
+#pragma unroll
+        for (int a = 0; a < 4; ++a) {
+          const float4v f4 = *reinterpret_cast<const float4v*>(fc + 8 * a);
+#pragma unroll
+          for (int c = 0; c < 4; ++c) sacc[4 * a + c] *= f4[c];
+        }
+      }
       // scores in the base-2 domain: s2 = (q.k) scale log2e - slope log2e (pos - j), one add and one fma each
       float sv[16];
       const float tile_bias = -sl2 * (float)(pos - kbase);
       // interior tile: every key is visible to every token of the tile, no masks to evaluate
-      const bool interior = !sink && t_off + 31 < cnt && kbase + 31 <= p0 && (window == 0 || p1 - kbase < window);
+      const bool interior = !sink && t_off + 31 < cnt && kbase + 31 <= p0 && kbase >= lo_p1;
       if (summ) {  // summaries: seen by count, no distance terms
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
@@ -545,7 +577,7 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
           const int j = kbase + (i & 3) + 8 * (i >> 2) + 4 * hf;
-          const bool seen = tok_ok && j < klimit && j <= pos && (window == 0 || pos - j < window || j < keep_first);
+          const bool seen = tok_ok && j < klimit && j <= pos && (j >= lo || j < keep_first);
           sv[i] = seen ? base2(sacc[i]) + (tile_bias + row_bias[i]) : -INFINITY;
         }
       }
@@ -603,8 +635,8 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
   if (!tok_ok || !head_ok) return;
   float scale_out = 1.0f / l;
   if (gate != nullptr) scale_out *= sigmoidf_(ldf(gate + n * gate_stride + h));
-  if (cross_out != nullptr) {
-    float* crow = cross_out + ((n * H + h) * G + vg) * (long)Dvr;
+  if (cross_out != nullptr || out32 != nullptr) {
+    float* crow = cross_out != nullptr ? cross_out + ((n * H + h) * G + vg) * (long)Dvr : out32 + (n * H + h) * (long)Dvr;
 #pragma unroll
     for (int t = 0; t < VT; ++t)
 #pragma unroll
@@ -638,6 +670,10 @@ struct ScalarExtras {
   const void* vsum = nullptr;
   int sum_shift = 0, sum_block = 1;
   float* cross_out = nullptr;
+  int chunk = 0;
+  const float* key_fac = nullptr;
+  int vrep = 1;
+  float* out32 = nullptr;
 };
 
 static void launch_scalar_attention(at::Tensor& out, const at::Tensor& q, const at::Tensor& kpool, const at::Tensor& vpool,
@@ -673,12 +709,13 @@ static void launch_scalar_attention(at::Tensor& out, const at::Tensor& q, const 
   else SCALAR_LAUNCH(RC_, false)
 #define SCALAR_LAUNCH(RC_, V8_)                                                                                     \
   hipLaunchKernelGGL((paged_attention_kernel<T, RC_, V8_>), dim3((unsigned)(N * G * chunks * VC)), dim3(64 * nwaves), smem,   \
-                     stream(), x.cross_out != nullptr ? (T*)nullptr : ptr<T>(out), ptr<T>(q), (long)q.stride(0), ptr<T>(kpool), ptr<T>(vpool),             \
+                     stream(), (x.cross_out != nullptr || x.out32 != nullptr) ? (T*)nullptr : ptr<T>(out), ptr<T>(q), (long)q.stride(0), ptr<T>(kpool), ptr<T>(vpool),             \
                      block_tables.data_ptr<int>(), (int)block_tables.stride(0), tok_seq.data_ptr<int>(),            \
                      positions.data_ptr<int>(), slp, gate.has_value() ? ptr<T>(*gate) : (const T*)nullptr, gstride, \
                      H, G, D, Dv, page_shift, (float)scale, (int)window, (int)keep_first, kvec,                      \
                      vvec_even & vvec_ok, (float)softcap, sink ? 1 : 0, vrow, vhead, x.sink_logits, x.dist_bias, x.dist_rows,      \
-                     (const T*)x.ksum, (const T*)x.vsum, x.sum_shift, x.sum_block, x.cross_out)
+                     (const T*)x.ksum, (const T*)x.vsum, x.sum_shift, x.sum_block, x.cross_out, x.chunk, x.key_fac,        \
+                     x.vrep, x.out32)
   SERVING_DISPATCH_ACT(q, T, {
     if (rc == 4) { SCALAR_CASE(4); }
     else if (rc == 2) { SCALAR_CASE(2); }
@@ -711,20 +748,23 @@ static bool launch_mfma_attention(at::Tensor& out, const at::Tensor& q, const at
     const int VC = x.cross_out != nullptr ? G : 1;
     const dim3 grid((unsigned)(qsplit ? num_tiles128 : num_tiles), (unsigned)G, (unsigned)((rep + nw - 1) / nw * VC));
     const int ds = D <= 32 ? 2 : D <= 48 ? 3 : D <= 64 ? 4 : D <= 96 ? 6 : 8, vt = (Dv + 31) / 32;
-    const size_t msmem = (size_t)2 * MFMA_TILES_PER_STEP * (32 * (ds * 16 + 8) + vt * 32 * 40) * sizeof(bf16s);
+    const size_t msmem = (size_t)2 * MFMA_TILES_PER_STEP *
+                         ((32 * (ds * 16 + 8) + vt * 32 * 40) * sizeof(bf16s) + (x.key_fac != nullptr ? 32 * sizeof(float) : 0));
 #define MFMA_CASE(DS_, VT_)                                                                                        \
   do {                                                                                                             \
     auto kfn = paged_attention_mfma_kernel<DS_, VT_>;                                                              \
     if (msmem > 65536) /* more dynamic LDS than a kernel gets without asking */                                    \
       (void)hipFuncSetAttribute((const void*)kfn, hipFuncAttributeMaxDynamicSharedMemorySize, (int)msmem);         \
     hipLaunchKernelGGL(kfn, grid, dim3(64 * nw), msmem, stream(),                                                 \
-                       x.cross_out != nullptr ? (bf16s*)nullptr : ptr<bf16s>(out), ptr<bf16s>(q),                  \
+                       (x.cross_out != nullptr || x.out32 != nullptr) ? (bf16s*)nullptr : ptr<bf16s>(out),         \
+                       ptr<bf16s>(q),                                                                              \
                        (long)q.stride(0), ptr<bf16s>(kpool), ptr<bf16s>(vpool), block_tables.data_ptr<int>(),      \
                        (int)block_tables.stride(0), cu.data_ptr<int>(), start.data_ptr<int>(), slp,                \
                        gate.has_value() ? ptr<bf16s>(*gate) : (const bf16s*)nullptr, gstride, H, G, D, Dv,         \
                        page_shift, (float)scale, (int)window, (int)keep_first, (float)softcap, sink ? 1 : 0,       \
                        qsplit, x.sink_logits, x.dist_bias, x.dist_rows, (const bf16s*)x.ksum,                      \
-                       (const bf16s*)x.vsum, x.sum_shift, x.sum_block, x.cross_out);                               \
+                       (const bf16s*)x.vsum, x.sum_shift, x.sum_block, x.cross_out, x.chunk, x.key_fac, x.vrep,    \
+                       x.out32);                                                                                   \
   } while (0)
 #define MFMA_ROW(DS_)                     \
   do {                                    \
@@ -793,16 +833,17 @@ at::Tensor paged_attention(at::Tensor q, at::Tensor kpool, at::Tensor vpool, at:
   return out;
 }
 
-// The split-key kernel with its optional extras, for prompt portions and decode tokens alike: a learned sink per
-// head, a per-distance bias table, block summaries ahead of the window, and (cross) every query head's weights
-// applied to every kv head's values, returned as float32 [N, H, G, Dv] for a talking-heads mix.
+// Attention with its optional extras, for prompt portions and decode tokens alike: a learned sink per
+// head, a per-distance bias table, block summaries ahead of the window, (cross) every query head's weights
+// applied to every kv head's values, returned as float32 [N, H, G, Dv] for a talking-heads mix, visibility inside blocks
+// of `chunk` positions, a factor per cached key, value pools with fewer heads than the key pool, float32 output.
 at::Tensor paged_attention_ext(at::Tensor q, at::Tensor kpool, at::Tensor vpool, at::Tensor block_tables, at::Tensor cu,
                                at::Tensor start, at::Tensor tok_seq, at::Tensor positions, double scale, int64_t window,
                                int64_t keep_first, c10::optional<at::Tensor> slopes, c10::optional<at::Tensor> gate,
                                double softcap, bool sink, c10::optional<at::Tensor> sink_logits,
                                c10::optional<at::Tensor> dist_bias, c10::optional<at::Tensor> ksum,
                                c10::optional<at::Tensor> vsum, int64_t sum_block, bool cross, int64_t num_tiles,
-                               int64_t num_tiles128) {
+                               int64_t num_tiles128, int64_t chunk, c10::optional<at::Tensor> key_fac, bool out_f32) {
   check_act(q, "q");
   TORCH_CHECK(softcap >= 0.0, "softcap must not be negative (0 = none)");
   TORCH_CHECK(q.dim() == 3 && q.stride(2) == 1 && q.stride(1) == q.size(2), "q must be [N, H, D] with dense rows");
@@ -813,11 +854,17 @@ at::Tensor paged_attention_ext(at::Tensor q, at::Tensor kpool, at::Tensor vpool,
   const long N = q.size(0);
   const int H = (int)q.size(1), D = (int)q.size(2);
   const int page = (int)kpool.size(1), G = (int)kpool.size(2), Dv = (int)vpool.size(3);
-  TORCH_CHECK(kpool.size(3) == D && vpool.size(2) == G && vpool.size(1) == page && vpool.size(0) == kpool.size(0));
+  const int Gv = (int)vpool.size(2);
+  TORCH_CHECK(kpool.size(3) == D && Gv > 0 && G % Gv == 0 && vpool.size(1) == page && vpool.size(0) == kpool.size(0),
+              "the value pool must have the key pool's pages and a divisor of its heads");
   TORCH_CHECK(H % G == 0 && Dv <= 512 && page > 0 && (page & (page - 1)) == 0);
   check_i32(block_tables, "block_tables"); check_i32(tok_seq, "tok_seq"); check_i32(positions, "positions");
   TORCH_CHECK(block_tables.dim() == 2 && tok_seq.numel() == N && positions.numel() == N);
-  TORCH_CHECK(window >= 0 && keep_first >= 0);
+  TORCH_CHECK(window >= 0 && keep_first >= 0 && chunk >= 0);
+  TORCH_CHECK(chunk == 0 || (window == 0 && keep_first == 0 && !ksum.has_value()),
+              "fixed blocks of positions take the place of a window");
+  TORCH_CHECK((Gv == G && !key_fac.has_value() && !out_f32) || (!cross && !ksum.has_value()),
+              "cross values and block summaries go with plain key/value heads");
   int page_shift = 0;
   while ((1 << page_shift) < page) ++page_shift;
   at::Tensor sl, sk, db;
@@ -834,6 +881,14 @@ at::Tensor paged_attention_ext(at::Tensor q, at::Tensor kpool, at::Tensor vpool,
     gstride = gate->stride(0);
   }
   ScalarExtras x;
+  x.chunk = (int)chunk;
+  x.vrep = G / Gv;
+  if (key_fac.has_value()) {
+    TORCH_CHECK(key_fac->is_cuda() && is_f32(*key_fac) && key_fac->is_contiguous() && key_fac->dim() == 3 &&
+                key_fac->size(0) == kpool.size(0) && key_fac->size(1) == page && key_fac->size(2) == G,
+                "key factors must be contiguous float32 [pages, page, G]");
+    x.key_fac = key_fac->data_ptr<float>();
+  }
   if (sink_logits.has_value()) {
     sk = f32c(*sink_logits);
     TORCH_CHECK(sk.is_cuda() && sk.numel() == H, "sink_logits must be [H]");
@@ -860,9 +915,11 @@ at::Tensor paged_attention_ext(at::Tensor q, at::Tensor kpool, at::Tensor vpool,
     x.ksum = ksum->data_ptr();
     x.vsum = vsum->data_ptr();
   }
-  at::Tensor out = cross ? at::empty({N, H, G, Dv}, q.options().dtype(at::kFloat)) : at::empty({N, H, Dv}, q.options());
+  at::Tensor out = cross ? at::empty({N, H, G, Dv}, q.options().dtype(at::kFloat))
+                         : at::empty({N, H, Dv}, out_f32 ? q.options().dtype(at::kFloat) : q.options());
   if (N == 0) return out;
   if (cross) x.cross_out = out.data_ptr<float>();
+  else if (out_f32) x.out32 = out.data_ptr<float>();
   if (num_tiles > 0 && is_bf16(q)) {  // prompt portions in bfloat16: the matrix-core kernel, extras in the base-2 domain
     check_i32(cu, "cu"); check_i32(start, "start");
     constexpr double LOG2E = 1.4426950408889634;

@@ -30,9 +30,11 @@ class KVCacheManager:
         layer_shapes: Optional[List[Optional[tuple]]] = None,
         layer_sources: Optional[List[Optional[int]]] = None,
         layer_summaries: Optional[List[Optional[int]]] = None,
+        layer_key_factors: Optional[List[bool]] = None,
     ):
         """``layer_shapes`` (optional) gives each layer its own
-        ``(kv_heads, key_dim, value_dim)`` or ``None`` for a layer that keeps no
+        ``(kv_heads, key_dim, value_dim)`` (or ``(key_heads, key_dim, value_dim,
+        value_heads)`` when key heads share value heads) or ``None`` for a layer that keeps no
         keys (a recurrent layer of a hybrid model); without it every layer gets
         ``(num_kv_heads, head_dim, head_dim)``. ``layer_sources`` (optional)
         names, for a layer that projects no keys of its own, the layer whose
@@ -45,7 +47,11 @@ class KVCacheManager:
         ``[num_blocks, rows, Hkv, D]`` with ``rows = summary_rows_per_page(block_size, P)``;
         summary ``b`` of a sequence lives in its page ``b // rows`` at row ``b % rows``,
         so the sequence's page table addresses both pools and freeing its pages
-        frees its summaries."""
+        frees its summaries.
+        ``layer_key_factors`` (optional) marks the layers that keep one float32 number per
+        token and key head beside the key (keys normed on reading): ``k_factors[i]``
+        ``[num_blocks, block_size, Hkv]``, addressed like the keys. A layer whose values
+        are its keys has a value size of 0; its attention reads ``k_pools[i]`` for both."""
         assert block_size & (block_size - 1) == 0, "block_size must be a power of two"
         self.num_layers = num_layers
         self.block_size = block_size
@@ -60,7 +66,7 @@ class KVCacheManager:
             for s in layer_shapes
         ]
         self.v_pools = [
-            None if s is None else torch.zeros(num_blocks, block_size, s[0], s[2], device=self.device, dtype=dtype)
+            None if s is None else torch.zeros(num_blocks, block_size, s[-1] if len(s) > 3 else s[0], s[2], device=self.device, dtype=dtype)
             for s in layer_shapes
         ]
         self.layer_sources = list(layer_sources) if layer_sources is not None else [None] * num_layers
@@ -85,6 +91,11 @@ class KVCacheManager:
             rows = summary_rows_per_page(block_size, int(P))
             self.k_summaries[i] = torch.zeros(num_blocks, rows, s[0], s[1], device=self.device, dtype=dtype)
             self.v_summaries[i] = torch.zeros(num_blocks, rows, s[0], s[2], device=self.device, dtype=dtype)
+        self.k_factors: List[Optional[torch.Tensor]] = [None] * num_layers
+        for i, marked in enumerate(layer_key_factors or []):
+            if marked:
+                self.k_factors[i] = torch.zeros(num_blocks, block_size, layer_shapes[i][0], device=self.device,
+                                                dtype=torch.float32)
         self._free: List[int] = list(range(num_blocks - 1, -1, -1))
         self._tables: Dict[int, List[int]] = {}  # seq id -> block ids
 

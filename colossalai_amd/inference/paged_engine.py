@@ -59,9 +59,10 @@ class ContinuousBatchEngine:
             shapes = model.kv_layer_shapes()
             sources = model.kv_layer_sources() if hasattr(model, "kv_layer_sources") else None
             summaries = model.kv_layer_summaries() if hasattr(model, "kv_layer_summaries") else None
+            factors = model.kv_layer_key_factors() if hasattr(model, "kv_layer_key_factors") else None
             self.kv = KVCacheManager(len(shapes), 0, 0, num_blocks=num_blocks, block_size=block_size,
                                      device=self.device, dtype=self.dtype, layer_shapes=shapes,
-                                     layer_sources=sources, layer_summaries=summaries)
+                                     layer_sources=sources, layer_summaries=summaries, layer_key_factors=factors)
             self.state = StateCacheManager(model.state_layer_buffers(), self.config.max_batch_size,
                                            device=self.device)
             self.rm = RequestManager(self.kv, max_batch_size=self.config.max_batch_size, state=self.state)
@@ -116,6 +117,9 @@ class ContinuousBatchEngine:
             want += [at + int(j) for j in w]
             at += len(toks)
         assert len(set(slots)) == len(slots), "a sequence appears twice in one step"
+        vocab = getattr(self.model.config, "vocab", None)
+        if vocab is not None and flat and not 0 <= min(flat) <= max(flat) < vocab:
+            raise ValueError(f"token ids must lie in 0 .. {vocab - 1}")
         batch = RaggedBatch.build(counts, starts, slots, self.device, tables, self.kv.block_size)
         tokens = torch.tensor(flat, dtype=torch.long, device=self.device)
         widx = torch.tensor(want, dtype=torch.long, device=self.device)

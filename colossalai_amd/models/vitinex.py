@@ -48,6 +48,7 @@ from ..ops.pair_rotary import pair_frequencies
 from ..ops.ragged import RaggedBatch
 from ..ops.routed_experts import grouped_topk_route, routed_expert_ffn
 from ..ops.short_conv import short_conv
+from .looped import layer_runs, parse_loop
 from .packed import PackedLinear
 from .registry import register_model
 
@@ -65,11 +66,8 @@ class VitinexConfig:
 
     @classmethod
     def from_dict(cls, d: dict) -> "VitinexConfig":
-        loop = d.get("loop")
-        if loop is not None:
-            loop = {k: int(loop[k]) for k in ("start", "stop", "times")}
         return cls(vocab=int(d["vocab"]), width=int(d["width"]), layers=list(d["layers"]),
-                   norm_eps=float(d["norm"]["eps"]), residual_mult=float(d.get("residual_mult", 1.0)), loop=loop)
+                   norm_eps=float(d["norm"]["eps"]), residual_mult=float(d.get("residual_mult", 1.0)), loop=parse_loop(d))
 
     def to_dict(self) -> dict:
         d = {"architecture": "Vitinex", "layers": self.layers, "norm": {"eps": self.norm_eps},
@@ -80,16 +78,7 @@ class VitinexConfig:
 
     def layer_runs(self):
         """The order in which layers run: ``(layer, pass number or None, first of its pass)``."""
-        n = len(self.layers)
-        lp = self.loop
-        if lp is None or lp["stop"] <= lp["start"] or lp["times"] < 1:
-            return [(i, None, False) for i in range(n)]
-        if not 0 <= lp["start"] < lp["stop"] <= n:
-            raise ValueError(f"loop {lp} does not fit {n} layers")
-        runs = [(i, None, False) for i in range(lp["start"])]
-        for t in range(lp["times"]):
-            runs += [(i, t, i == lp["start"]) for i in range(lp["start"], lp["stop"])]
-        return runs + [(i, None, False) for i in range(lp["stop"], n)]
+        return layer_runs(len(self.layers), self.loop)
 
 
 def _vec(n, value=1.0):
@@ -114,6 +103,7 @@ class VitinexLatentAttention(nn.Module):
         self.uv = nn.Parameter(torch.randn(self.H, self.Dv, self.rank) * self.rank ** -0.5)
         self.o = nn.Linear(self.H * self.Dv, width, bias=False)
         self.register_buffer("freqs", pair_frequencies(self.rot_base, self.rot_dims), persistent=False)
+        self.register_buffer("uv_t", None, persistent=False)  # uv with its last two axes swapped, for decode steps
 
     def kv_shape(self):
         """One key head holding the latent and the shared rotated part; the values are a view of it."""
@@ -128,7 +118,8 @@ class VitinexLatentAttention(nn.Module):
         latent_kv_write(p["dkv"], self.dkv_norm, self.eps, self.freqs, pool, batch)
         cq = grouped_rms_norm(p["dq"], self.dq_norm, 1, self.eps, None, h.dtype)
         q = self.uq(cq).view(N, self.H, self.D + self.R)
-        o = latent_attention(q, self.uk, self.uv, pool, batch, self.scale, self.freqs, self.rank, p["g"])
+        o = latent_attention(q, self.uk, self.uv, pool, batch, self.scale, self.freqs, self.rank, p["g"],
+                             w_uv_t=self.uv_t)
         return self.o(o)
 
 
@@ -359,6 +350,7 @@ class VitinexForCausalLM(nn.Module):
                 put(m.uq.weight, get(a + "uq"))
                 put(m.uk, get(a + "uk").view(m.H, m.D, m.rank))
                 put(m.uv, get(a + "uv").view(m.H, m.Dv, m.rank))
+                m.uv_t = m.uv.detach().transpose(1, 2).contiguous()
                 put(m.o.weight, get(a + "o"))
             else:
                 put(m.in_proj.weight, get(a + "in"))

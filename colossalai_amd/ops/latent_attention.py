@@ -23,6 +23,10 @@ latents of the step's sequences (cached tokens included) into per-head keys
 multi-head attention over it (``expanded_attention``); the cache itself still
 holds latents only.
 
+The rotated part is optional (``freqs=None``, ``R = 0``: positions enter through the
+mask alone). With a sliding window the per-head form lays out only what the step's
+queries can see.
+
 ``latent_kv_write`` forms a step's rows (norm of the latent part, rotation of
 the shared key part) and scatters them into the pool in one launch.
 """
@@ -49,18 +53,22 @@ EXPAND_MAX_HEAD = 128
 
 def latent_kv_write_ref(dkv, norm_w, eps: float, freqs, pool, batch: RaggedBatch):
     rank = norm_w.numel()
-    c = grouped_rms_norm_ref(dkv[:, :rank], norm_w, 1, eps, None, torch.float32)
-    r = rotate_pairs_ref(dkv[:, None, rank:].float(), batch.positions, freqs)[:, 0]
+    row = grouped_rms_norm_ref(dkv[:, :rank], norm_w, 1, eps, None, torch.float32)
+    if freqs is not None:
+        row = torch.cat([row, rotate_pairs_ref(dkv[:, None, rank:].float(), batch.positions, freqs)[:, 0]], -1)
     rows = batch.kv_rows.long()
-    pool.view(-1, pool.shape[-1])[rows] = torch.cat([c, r], -1).to(pool.dtype)
+    pool.view(-1, pool.shape[-1])[rows] = row.to(pool.dtype)
 
 
 def latent_kv_write(dkv, norm_w, eps: float, freqs, pool, batch: RaggedBatch):
     """dkv [N, rank + R] (rows may be strided): the first ``rank`` channels are RMS-normed with ``norm_w`` (float32
-    statistics), the last ``R`` rotated pair-wise by the tokens' positions; the row goes to ``batch.kv_rows`` of
+    statistics), the last ``R`` rotated pair-wise by the tokens' positions (``freqs=None``: there are none); the row goes to ``batch.kv_rows`` of
     ``pool`` [pages, page_size, 1, rank + R]."""
     assert pool.shape[2] == 1 and pool.shape[3] == dkv.shape[1]
+    assert freqs is not None or norm_w.numel() == dkv.shape[1]
     if use_hip(dkv):
+        if freqs is None:
+            freqs = dkv.new_empty(0, dtype=torch.float32)
         serving_kernels().latent_kv_write(dkv, norm_w, eps, freqs, batch.positions, pool, batch.kv_rows)
         return
     latent_kv_write_ref(dkv, norm_w, eps, freqs, pool, batch)
@@ -73,15 +81,18 @@ def absorb_queries(q, w_uk, positions, freqs, rank: int):
     D = w_uk.shape[1]
     out = torch.empty(N, H, rank + DR - D, dtype=q.dtype, device=q.device)
     torch.bmm(q[:, :, :D].transpose(0, 1), w_uk, out=out[:, :, :rank].transpose(0, 1))
-    rotate_pairs(q[:, :, D:], positions, freqs, out=out[:, :, rank:])
+    if freqs is not None:
+        rotate_pairs(q[:, :, D:], positions, freqs, out=out[:, :, rank:])
     return out
 
 
-def expand_values(o, w_uv):
-    """o [N, H, rank] (weighted sums of latents), w_uv [H, Dv, rank] -> [N, H * Dv]."""
+def expand_values(o, w_uv, w_uv_t=None):
+    """o [N, H, rank] (weighted sums of latents), w_uv [H, Dv, rank] -> [N, H * Dv]. ``w_uv_t`` [H, rank, Dv]: the same
+    matrices transposed, when the caller keeps them (the right operand of the batched product must not be a transposed
+    view)."""
     N, H, _ = o.shape
     out = torch.empty(N, H, w_uv.shape[1], dtype=o.dtype, device=o.device)
-    torch.bmm(o.transpose(0, 1), w_uv.transpose(1, 2), out=out.transpose(0, 1))
+    torch.bmm(o.transpose(0, 1), w_uv.transpose(1, 2).contiguous() if w_uv_t is None else w_uv_t, out=out.transpose(0, 1))
     return out.view(N, -1)
 
 
@@ -100,14 +111,17 @@ def expanded_attention(q, w_uk, w_uv, pool, batch: RaggedBatch, scale: float, fr
     un-rotated (its rotated part is turned in place). Returns [N, H * Dv]."""
     N, H, DR = q.shape
     D, Dv = w_uk.shape[1], w_uv.shape[1]
-    rows, tables, total = batch.dense_context()
+    rows, tables, total = batch.dense_context(window if keep_first == 0 else 0)
     ctx = pool.view(-1, pool.shape[-1]).index_select(0, rows)                     # [total, rank + R]
-    keys = torch.empty(total, H, DR, dtype=q.dtype, device=q.device)
-    torch.bmm(ctx[:, :rank].unsqueeze(0).expand(H, total, rank), w_uk.transpose(1, 2),
-              out=keys[:, :, :D].transpose(0, 1))
-    keys[:, :, D:] = ctx[:, None, rank:]
     values = torch.mm(ctx[:, :rank], w_uv.reshape(H * Dv, rank).t())              # [total, H * Dv]
-    rotate_pairs(q[:, :, D:], batch.positions, freqs, out=q[:, :, D:])
+    if freqs is None:
+        keys = torch.mm(ctx, w_uk.reshape(H * D, rank).t())                       # [total, H * D]
+    else:
+        keys = torch.empty(total, H, DR, dtype=q.dtype, device=q.device)
+        torch.bmm(ctx[:, :rank].unsqueeze(0).expand(H, total, rank), w_uk.transpose(1, 2).contiguous(),
+                  out=keys[:, :, :D].transpose(0, 1))
+        keys[:, :, D:] = ctx[:, None, rank:]
+        rotate_pairs(q[:, :, D:], batch.positions, freqs, out=q[:, :, D:])
     ps = batch.page_size
     dense = dataclasses.replace(batch, block_tables=tables, kv_rows=None, _dense=None)
     o = paged_attention(q, keys.view(total // ps, ps, H, DR), values.view(total // ps, ps, H, Dv), dense, scale,
@@ -116,11 +130,11 @@ def expanded_attention(q, w_uk, w_uv, pool, batch: RaggedBatch, scale: float, fr
 
 
 def latent_attention(q, w_uk, w_uv, pool, batch: RaggedBatch, scale: float, freqs, rank: int,
-                     gate: Optional[torch.Tensor] = None, window: int = 0, keep_first: int = 0):
+                     gate: Optional[torch.Tensor] = None, window: int = 0, keep_first: int = 0, w_uv_t=None):
     """Causal softmax attention of a ragged step over latent rows already in ``pool``. q [N, H, D + R] un-rotated;
-    ``gate`` [N, H] logits of a per-head sigmoid output gate. Returns [N, H * Dv]."""
+    ``gate`` [N, H] logits of a per-head sigmoid output gate; ``freqs=None``: no rotated part. Returns [N, H * Dv]."""
     if expands(q, w_uk, w_uv, batch):
         return expanded_attention(q, w_uk, w_uv, pool, batch, scale, freqs, rank, gate, window, keep_first)
     qa = absorb_queries(q, w_uk, batch.positions, freqs, rank)
     o = paged_attention(qa, pool, pool[..., :rank], batch, scale, window, keep_first, None, gate)
-    return expand_values(o, w_uv)
+    return expand_values(o, w_uv, w_uv_t)

@@ -25,11 +25,19 @@ keys (``paged_kv_write`` runs first). Masking and bias are parameters:
   positions ``[bP, bP + P)`` that ends at or before ``i - w``; the summaries are
   the means of the block's cached keys and values (``paged_pool_write``), they
   share the softmax with the window's keys and get no distance terms;
+* optional *fixed blocks of positions*: with ``chunk`` a query at ``i`` sees the
+  keys from ``i - i % chunk`` on (blocks are counted from position 0 of the
+  sequence) instead of a window;
+* an optional float32 *factor per cached key* (``key_factors`` [pages, page, G]):
+  the score of a key is multiplied by it, so that keys which are normed on
+  reading can be cached as projected (``ops/normed_keys.py``);
+* a value pool with fewer heads than the key pool: consecutive key heads share a
+  value head (two attention maps over the same values are two key heads);
 * optional *talking heads*: the softmax weights of the heads are mixed,
   ``p'_h = sum_g talk[h, g] p_g``, before head ``h`` applies them to the values
   of its own key/value head.
 
-Scores, softmax weights and the accumulation are float32. Key and value head
+``out_dtype=torch.float32`` hands the result back unrounded. Scores, softmax weights and the accumulation are float32. Key and value head
 sizes may differ; query head ``h`` reads key/value head ``h // (H / G)``.
 """
 
@@ -128,9 +136,10 @@ def paged_attention_ref(q, kpool, vpool, batch: RaggedBatch, scale: float, windo
                         slopes: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
                         softcap: float = 0.0, sink: bool = False, sink_logits: Optional[torch.Tensor] = None,
                         dist_bias: Optional[torch.Tensor] = None, pooled: Optional[Tuple] = None,
-                        talk: Optional[torch.Tensor] = None):
+                        talk: Optional[torch.Tensor] = None, chunk: int = 0,
+                        key_factors: Optional[torch.Tensor] = None, out_dtype=None):
     N, H, D = q.shape
-    G, Dv = vpool.shape[2], vpool.shape[3]
+    G, Gv, Dv = kpool.shape[2], vpool.shape[2], vpool.shape[3]
     ps = kpool.shape[1]
     out = torch.empty(N, H, Dv, dtype=torch.float32, device=q.device)
     for i in range(batch.num_seqs):
@@ -138,11 +147,13 @@ def paged_attention_ref(q, kpool, vpool, batch: RaggedBatch, scale: float, windo
         L = s0 + hi - lo
         pages = batch.block_tables[i, : (L + ps - 1) // ps].long()
         kk = kpool[pages].reshape(-1, G, D)[:L].float().repeat_interleave(H // G, 1)   # [L, H, D]
-        vv = vpool[pages].reshape(-1, G, Dv)[:L].float().repeat_interleave(H // G, 1)
+        vv = vpool[pages].reshape(-1, Gv, Dv)[:L].float().repeat_interleave(H // Gv, 1)
         qi = torch.arange(s0, L, device=q.device)[:, None]
         kj = torch.arange(L, device=q.device)[None, :]
         dist = (qi - kj).float()
         s = torch.einsum("nhd,lhd->hnl", q[lo:hi].float(), kk) * scale
+        if key_factors is not None:
+            s = s * key_factors[pages].reshape(-1, G)[:L].repeat_interleave(H // G, 1).t()[:, None, :]
         if softcap > 0:
             s = softcap * torch.tanh(s / softcap)
         if slopes is not None:
@@ -153,6 +164,8 @@ def paged_attention_ref(q, kpool, vpool, batch: RaggedBatch, scale: float, windo
         seen = kj <= qi
         if window > 0:
             seen = seen & ((qi - kj < window) | (kj < keep_first))
+        if chunk > 0:
+            seen = seen & (kj >= qi - qi % chunk)
         s = s.masked_fill(~seen, float("-inf"))
         n_sum = 0
         if pooled is not None:  # one summary per block that ends at or before i - window, ahead of the keys
@@ -180,27 +193,33 @@ def paged_attention_ref(q, kpool, vpool, batch: RaggedBatch, scale: float, windo
         out[lo:hi] = torch.einsum("hnl,lhv->nhv", p, vv)
     if gate is not None:
         out = out * torch.sigmoid(gate.float())[:, :, None]
-    return out.to(q.dtype)
+    return out.to(out_dtype or q.dtype)
 
 
 def paged_attention(q, kpool, vpool, batch: RaggedBatch, scale: float, window: int = 0, keep_first: int = 0,
                     slopes: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
                     softcap: float = 0.0, sink: bool = False, sink_logits: Optional[torch.Tensor] = None,
                     dist_bias: Optional[torch.Tensor] = None, pooled: Optional[Tuple] = None,
-                    talk: Optional[torch.Tensor] = None):
-    """q [N, H, D]; returns [N, H, Dv] in q's dtype. ``window == 0`` means no
-    window; ``gate`` [N, H] logits or None; ``softcap == 0`` means no cap;
+                    talk: Optional[torch.Tensor] = None, chunk: int = 0,
+                    key_factors: Optional[torch.Tensor] = None, out_dtype=None):
+    """q [N, H, D]; returns [N, H, Dv] in q's dtype (or ``out_dtype``, float32 only). ``window == 0`` means no
+    window and ``chunk == 0`` no fixed blocks (at most one of them); ``gate`` [N, H] logits or None; ``softcap == 0`` means no cap;
     ``sink_logits`` [H] float32; ``dist_bias`` [rows, H] float32; ``pooled`` =
     (key summaries, value summaries, block) needs a window; ``talk`` [H, H]."""
     assert pooled is None or window > 0, "block summaries stand for what a window no longer shows"
-    if use_hip(q) and (sink_logits is not None or dist_bias is not None or pooled is not None or talk is not None):
+    assert chunk == 0 or (window == 0 and keep_first == 0 and pooled is None)
+    assert out_dtype in (None, q.dtype, torch.float32)
+    plain = chunk == 0 and key_factors is None and kpool.shape[2] == vpool.shape[2] and out_dtype in (None, q.dtype)
+    assert plain or (pooled is None and talk is None)
+    if use_hip(q) and not (plain and sink_logits is None and dist_bias is None and pooled is None and talk is None):
         # With talking heads the kernels hand back every query head's weights applied to every key/value head's
         # values, O[n, g, c] (float32): the mix is linear, so out[n, h] = sum_g talk[h, g] O[n, g, kv(h)]
         ksum, vsum, block = pooled if pooled is not None else (None, None, 0)
         o = serving_kernels().paged_attention_ext(q, kpool, vpool, batch.block_tables, batch.cu, batch.start,
                                                   batch.tok_seq, batch.positions, scale, window, keep_first, slopes,
                                                   gate, float(softcap), bool(sink), sink_logits, dist_bias, ksum, vsum,
-                                                  int(block), talk is not None, batch.num_tiles32, batch.num_tiles128)
+                                                  int(block), talk is not None, batch.num_tiles32, batch.num_tiles128, int(chunk),
+                                                  key_factors, out_dtype == torch.float32)
         if talk is None:
             return o
         return serving_kernels().talk_mix(o, talk, q.dtype)
@@ -210,4 +229,4 @@ def paged_attention(q, kpool, vpool, batch: RaggedBatch, scale: float, window: i
                                                  slopes, gate, batch.num_tiles32, float(softcap), bool(sink),
                                                  batch.num_tiles128)
     return paged_attention_ref(q, kpool, vpool, batch, scale, window, keep_first, slopes, gate, softcap, sink,
-                               sink_logits, dist_bias, pooled, talk)
+                               sink_logits, dist_bias, pooled, talk, chunk, key_factors, out_dtype)
