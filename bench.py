@@ -29,11 +29,13 @@ def parse_args():
     p.add_argument("--gpus", type=int, default=1)
     p.add_argument("--steps", type=int, default=5)
     p.add_argument("--warmup", type=int, default=2)
-    p.add_argument("--workload", type=str, default="train", choices=["train", "serve-hybrid", "serve-moe", "serve-latent", "serve-pooled"],
+    p.add_argument("--workload", type=str, default="train", choices=["train", "serve-hybrid", "serve-moe", "serve-latent", "serve-pooled",
+                                                                       "serve-streams"],
                    help="train: the headline training step (default). serve-hybrid / serve-moe / serve-latent / "
-                        "serve-pooled: prefill/decode tokens/s of the Kipirax hybrid / the Mubutar routed-experts model / "
+                        "serve-pooled / serve-streams: prefill/decode tokens/s of the Kipirax hybrid / the Mubutar routed-experts model / "
                         "the Vitinex latent-attention + state-space model / the Tarulix window + block-summary + "
-                        "selective-scan model next to a Llama of equal size (the last two also next to Mubutar), all "
+                        "selective-scan model / the Bekulix multi-stream model next to a Llama of equal size (the last three "
+                        "also next to Mubutar, the last also next to Vitinex), all "
                         "through the continuous-batching engine")
     p.add_argument("--serve-sizes", type=str, default="w2048,w4096")
     p.add_argument("--model", type=str, default="llama-7b")
@@ -70,7 +72,7 @@ def serve_comparison(args, kind):
 
 def main():
     args = parse_args()
-    if args.workload in ("serve-hybrid", "serve-moe", "serve-latent", "serve-pooled"):
+    if args.workload in ("serve-hybrid", "serve-moe", "serve-latent", "serve-pooled", "serve-streams"):
         return serve_comparison(args, args.workload.split("-")[1])
     import colossalai_amd
     from colossalai_amd.models import LLAMA_CONFIGS, LlamaForCausalLM, llama_flops_per_token

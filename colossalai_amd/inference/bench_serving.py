@@ -1,13 +1,15 @@
 """Serving throughput of the ragged-step models next to a Llama of equal width,
 depth and per-token work, all through ``ContinuousBatchEngine``: prefill tokens/s
 of one long prompt and decode tokens/s of a batch of running sequences. Random
-weights, synthetic tokens. Four comparisons: the Kipirax hybrid (paged window
+weights, synthetic tokens. Five comparisons: the Kipirax hybrid (paged window
 attention + recurrent state), Mubutar (sink-softmax attention with shared
 keys, routed experts), Vitinex (latent attention + state-space layers in a
-looped block, routed experts) and Tarulix (windowed attention with a distance
+looped block, routed experts), Tarulix (windowed attention with a distance
 table and a learned sink; window + block summaries + talking heads beside a
-selective scan; gated experts with identity experts), the last two also next to
-Mubutar, whose kernels are the closest.
+selective scan; gated experts with identity experts) and Bekulix (parallel residual
+streams; attention whose values are its keys, chunked differential attention and
+windowed latent attention; looped block), the last three also next to Mubutar, whose
+kernels are the closest, and Bekulix also next to Vitinex.
 """
 
 import json
@@ -16,12 +18,13 @@ from typing import Dict, List
 
 import torch
 
-from ..models import (KipiraxConfig, KipiraxForCausalLM, LlamaConfig, LlamaForCausalLM, MubutarConfig,
+from ..models import (BekulixConfig, BekulixForCausalLM, KipiraxConfig, KipiraxForCausalLM, LlamaConfig, LlamaForCausalLM, MubutarConfig,
                       MubutarForCausalLM, TarulixConfig, TarulixForCausalLM, VitinexConfig, VitinexForCausalLM)
 from .config import InferenceConfig
 from .paged_engine import ContinuousBatchEngine
 
 __all__ = ["SIZES", "hybrid_config", "llama_config", "moe_config", "latent_config", "pooled_config",
+           "streams_config",
            "run_serving_comparison"]
 
 # width, layers, heads, kv_heads, head size, vocab
@@ -113,6 +116,21 @@ def pooled_config(s: dict, experts: int = 32, top: int = 6, window: int = 1024, 
     return TarulixConfig(vocab=s["vocab"], width=W, layers=layers, norm_eps=1e-6)
 
 
+def streams_config(s: dict, window: int = 1024, streams: int = 4) -> BekulixConfig:
+    """As many layer runs as the size has layers, the first two looped twice: full attention over shared keys/values,
+    chunked differential attention (two maps of half the head size each over blocks of ``window`` positions) and
+    windowed latent attention in turn, Llama's head sizes and feed-forward (ReLU), a latent of twice the head size."""
+    W, H, G, D = s["width"], s["heads"], s["kv_heads"], s["dim"]
+    att = dict(dim=D, heads=H, kv_heads=G, vdim=D, scale=D ** -0.5, q_temp=dict(coef=0.1, every=512))
+    dif = dict(dim=D // 2, heads=H, kv_heads=G, vdim=D, scale=(D // 2) ** -0.5, diff=0.4, mask=dict(size=window))
+    lat = dict(dim=D, heads=H, vdim=D, kv_rank=2 * D, scale=D ** -0.5, mask=dict(size=window))
+    kinds = [("attention", att), ("attention_2", dif), ("latent_attention", lat)]
+    layers = [dict(type=kinds[i % 3][0], mixer=kinds[i % 3][1], mlp=dict(kind="dense", ff=_inter(W)))
+              for i in range(s["layers"] - 2)]
+    return BekulixConfig(vocab=s["vocab"], width=W, layers=layers, norm_eps=1e-6, streams=streams,
+                         loop=dict(start=0, stop=2, times=2))
+
+
 def llama_config(s: dict, max_positions: int) -> LlamaConfig:
     # gate/up/down of 8/3 W carry the parameters of the hybrid's up/down of 4 W
     inter = _inter(s["width"])
@@ -192,6 +210,17 @@ def _pooled_numbers(s: dict, prompt: int, batch: int, context: int, steps: int) 
     return _ragged_numbers(model, cfg.vocab, prompt, batch, context, steps)
 
 
+def _streams_numbers(s: dict, prompt: int, batch: int, context: int, steps: int) -> Dict[str, float]:
+    cfg = streams_config(s)
+    model = BekulixForCausalLM(cfg).serving_dtype(torch.bfloat16).to("cuda").eval()
+    with torch.no_grad():
+        for p in model.parameters():
+            if p.dtype == torch.bfloat16:
+                p.normal_(0, 0.02)
+    model.prepare()
+    return _ragged_numbers(model, cfg.vocab, prompt, batch, context, steps)
+
+
 def _ragged_numbers(model, vocab: int, prompt: int, batch: int, context: int, steps: int) -> Dict[str, float]:
     page = 64
     blocks = max(prompt, batch * (context + steps + page)) // page + batch + 2
@@ -247,15 +276,18 @@ def _llama_numbers(s: dict, prompt: int, batch: int, context: int, steps: int) -
 
 def run_serving_comparison(sizes: List[str], prompt: int = 4096, batch: int = 16, context: int = 1024,
                            steps: int = 32, kind: str = "hybrid") -> dict:
-    """``kind``: "hybrid" (Kipirax), "moe" (Mubutar), "latent" (Vitinex) or "pooled" (Tarulix), each next to
-    Llama; "latent" and "pooled" also next to Mubutar."""
-    ours = {"hybrid": _hybrid_numbers, "moe": _moe_numbers, "latent": _latent_numbers, "pooled": _pooled_numbers}[kind]
+    """``kind``: "hybrid" (Kipirax), "moe" (Mubutar), "latent" (Vitinex), "pooled" (Tarulix) or "streams" (Bekulix),
+    each next to Llama; the last three also next to Mubutar, "streams" also next to Vitinex."""
+    ours = {"hybrid": _hybrid_numbers, "moe": _moe_numbers, "latent": _latent_numbers, "pooled": _pooled_numbers,
+            "streams": _streams_numbers}[kind]
     out = {}
     for name in sizes:
         s = SIZES[name]
         out[name] = {kind: ours(s, prompt, batch, context, steps)}
-        if kind in ("latent", "pooled"):
+        if kind in ("latent", "pooled", "streams"):
             out[name]["moe"] = _moe_numbers(s, prompt, batch, context, steps)
+        if kind == "streams":
+            out[name]["latent"] = _latent_numbers(s, prompt, batch, context, steps)
         out[name]["llama"] = _llama_numbers(s, prompt, batch, context, steps)
         out[name]["shape"] = dict(s, prompt=prompt, batch=batch, context=context)
     return out
