@@ -447,6 +447,44 @@ __global__ __launch_bounds__(256) void query_norm_key_write_kernel(
   }
 }
 
+// The same for head sizes that are multiples of 8 (up to 512): a lane holds 8 neighbouring channels, 2^lane_shift lanes a
+// head, so a wave does several heads with 16/32-byte loads and stores.
+template <typename T>
+__global__ __launch_bounds__(256) void query_norm_key_write_vec_kernel(
+    T* __restrict__ out, T* __restrict__ kpool, float* __restrict__ kfac, const T* __restrict__ q, long qs,
+    const T* __restrict__ k, long ks, const float* __restrict__ w, const int* __restrict__ positions,
+    const int* __restrict__ rows, long units, int H, int G, int D, float eps, float coef, double every, int lane_shift) {
+  const long t = (long)blockIdx.x * blockDim.x + threadIdx.x;
+  const long unit = t >> lane_shift;
+  const bool live = unit < units;     // lanes beyond the last head still take part in the shuffles
+  const int d = ((int)t & ((1 << lane_shift) - 1)) * 8;
+  const bool mine = live && d < D;
+  const long n = live ? unit / (H + G) : 0;
+  const int hd = live ? (int)(unit % (H + G)) : 0;
+  const bool query = hd < H;
+  float v[8], ssq = 0.0f;
+  if (mine) {
+    load8(query ? q + n * qs + (long)hd * D + d : k + n * ks + (long)(hd - H) * D + d, v);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ssq += v[e] * v[e];
+  }
+  for (int off = 1 << lane_shift >> 1; off > 0; off >>= 1) ssq += __shfl_xor(ssq, off);
+  if (!mine) return;
+  const float inv = 1.0f / sqrtf(ssq / (float)D + eps);
+  if (query) {
+    float f = inv, wv[8];
+    if (every > 0.0) f *= 1.0f + coef * logf((float)(floor((double)(positions[n] + 1) / every) + 1.0));
+    load8(w + d, wv);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] *= f * wv[e];
+    store8(out + (n * H + hd) * (long)D + d, v);
+  } else {
+    const long row = (long)rows[n] * G + (hd - H);
+    store8(kpool + row * D + d, v);
+    if (d == 0) kfac[row] = inv;
+  }
+}
+
 at::Tensor query_norm_key_write(at::Tensor q, at::Tensor k, at::Tensor weight, double eps, double coef, double every,
                                 at::Tensor positions, at::Tensor kpool, at::Tensor kfac, at::Tensor rows) {
   check_act(q, "q"); check_act(k, "k");
@@ -467,6 +505,20 @@ at::Tensor query_norm_key_write(at::Tensor q, at::Tensor k, at::Tensor weight, d
   at::Tensor out = at::empty({N, H, D}, q.options());
   const long units = N * (H + G);
   if (units == 0) return out;
+  auto al16 = [](const at::Tensor& t) { return reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0; };  // two 16-byte loads
+  if (D % 8 == 0 && q.stride(0) % 8 == 0 && k.stride(0) % 8 == 0 && al16(q) && al16(k) && al16(out) && al16(kpool) && al16(w)) {
+    int lane_shift = 0;
+    while ((8 << lane_shift) < D) ++lane_shift;
+    const long threads = units << lane_shift;
+    SERVING_DISPATCH_ACT(q, T, {
+      hipLaunchKernelGGL(query_norm_key_write_vec_kernel<T>, dim3((unsigned)((threads + 255) / 256)), dim3(256), 0, stream(),
+                         ptr<T>(out), ptr<T>(kpool), kfac.data_ptr<float>(), ptr<T>(q), (long)q.stride(0), ptr<T>(k),
+                         (long)k.stride(0), w.data_ptr<float>(), positions.data_ptr<int>(), rows.data_ptr<int>(), units, H,
+                         G, D, (float)eps, (float)coef, every, lane_shift);
+    });
+    HIP_CHECK_LAST();
+    return out;
+  }
   const dim3 grid((unsigned)((units + 3) / 4));
 #define QNK_LAUNCH(PER_)                                                                                            \
   hipLaunchKernelGGL((query_norm_key_write_kernel<T, PER_>), grid, dim3(256), 0, stream(), ptr<T>(out), ptr<T>(kpool), \

@@ -17,7 +17,7 @@
 // the 64-key blocks. Phase 2: lane = value channel, the block's weights and
 // pool rows are broadcast from LDS. A prompt portion and a decode token run
 // the same code, so a position's result depends on nothing but the pages.
-#include "serving_common.h"
+#include "paged_attention.h"
 
 namespace cai {
 namespace serving {
@@ -26,19 +26,8 @@ constexpr int ATT_WAVES = 16;  // most waves of a block: they split the key bloc
 constexpr int RC_MAX = 4;      // most query heads of a kv head's group that one block handles together
 constexpr int MFMA_TILES_PER_STEP = 2;  // 32-key tiles the matrix-core kernel stages and multiplies between two barriers
 
-template <int CTRL>
-DEV_INLINE float dpp_add(float v) {
-  const int moved = __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xf, 0xf, false);
-  return v + __builtin_bit_cast(float, moved);
-}
 // sum over the 8 adjacent lanes that share a key (quad xor 1, quad xor 2, half-row mirror)
 DEV_INLINE float reduce8(float v) { return dpp_add<0x141>(dpp_add<0x4E>(dpp_add<0xB1>(v))); }
-
-// First position a query at `pos` sees: its block of `chunk` positions, its window, or position 0.
-DEV_INLINE int first_visible(int pos, int window, int chunk) {
-  if (chunk > 0) return pos - pos % chunk;
-  return window > 0 ? max(0, pos - window + 1) : 0;
-}
 
 // Scalar kernel (decode tokens, float32 serving, shapes the MFMA kernel does not take).
 // One block per (token, kv head, group of up to RC query heads of that kv head): keys and
@@ -661,21 +650,6 @@ __global__ __launch_bounds__(256) void paged_attention_mfma_kernel(
     }
 }
 
-// What the split-key kernel takes beyond the common parameters (all optional).
-struct ScalarExtras {
-  const float* sink_logits = nullptr;
-  const float* dist_bias = nullptr;
-  int dist_rows = 0;
-  const void* ksum = nullptr;
-  const void* vsum = nullptr;
-  int sum_shift = 0, sum_block = 1;
-  float* cross_out = nullptr;
-  int chunk = 0;
-  const float* key_fac = nullptr;
-  int vrep = 1;
-  float* out32 = nullptr;
-};
-
 static void launch_scalar_attention(at::Tensor& out, const at::Tensor& q, const at::Tensor& kpool, const at::Tensor& vpool,
                                     const at::Tensor& block_tables, const at::Tensor& tok_seq, const at::Tensor& positions,
                                     const float* slp, const c10::optional<at::Tensor>& gate, long gstride, double scale,
@@ -684,6 +658,9 @@ static void launch_scalar_attention(at::Tensor& out, const at::Tensor& q, const 
   const long N = q.size(0);
   const int H = (int)q.size(1), D = (int)q.size(2);
   const int G = (int)kpool.size(2), Dv = (int)vpool.size(3);
+  if (launch_row_attention(out, q, kpool, vpool, block_tables, tok_seq, positions, slp, gate, gstride, scale, window,
+                           keep_first, softcap, sink, page_shift, vrow, vhead, x))
+    return;
   const int VC = x.cross_out != nullptr ? G : 1;
   const int Dp = (D + 7) & ~7;
   const int R = H / G;

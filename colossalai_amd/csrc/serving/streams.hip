@@ -187,8 +187,9 @@ c10::optional<at::Tensor> streams_update(at::Tensor x, at::Tensor y, at::Tensor 
   return h;
 }
 
-// One block per token: table row tokens[n] -> all S streams, and rms_norm((sum_s in[s]) * row) * w.
-template <typename TE>
+// One block per token: table row tokens[n] -> all S streams, and rms_norm((sum_s in[s]) * row) * w. V channels per
+// thread and step (4: the width is a multiple of 4 and every row 16-byte aligned); the row is read again for the norm.
+template <typename TE, int V>
 __global__ __launch_bounds__(256) void streams_start_kernel(TE* __restrict__ h, float* __restrict__ x,
                                                             const TE* __restrict__ table, const long* __restrict__ tokens,
                                                             const float* __restrict__ w_in, const float* __restrict__ w,
@@ -199,15 +200,33 @@ __global__ __launch_bounds__(256) void streams_start_kernel(TE* __restrict__ h, 
   float* xr = x + row * S * (long)W;
   float ssq = 0.0f, total = 0.0f;
   for (int s = 0; s < S; ++s) total += w_in[s];
-  for (int i = threadIdx.x; i < W; i += blockDim.x) {
-    const float e = ldf(er + i);
-    for (int s = 0; s < S; ++s) xr[(long)s * W + i] = e;
-    const float u = total * e;
-    ssq += u * u;
+#pragma unroll 2
+  for (int i = threadIdx.x * V; i < W; i += blockDim.x * V) {
+    float e[V];
+    if constexpr (V == 4) load4(er + i, e);
+    else e[0] = ldf(er + i);
+#pragma unroll
+    for (int k = 0; k < V; ++k) ssq += (total * e[k]) * (total * e[k]);
+    for (int s = 0; s < S; ++s) {
+      if constexpr (V == 4) store4(xr + (long)s * W + i, e);
+      else xr[(long)s * W + i] = e[0];
+    }
   }
   ssq = block_reduce_sum(ssq, red);
-  const float inv = 1.0f / sqrtf(ssq / (float)W + eps);
-  for (int i = threadIdx.x; i < W; i += blockDim.x) stf(h + row * (long)W + i, total * ldf(er + i) * inv * w[i]);
+  const float inv = total / sqrtf(ssq / (float)W + eps);
+#pragma unroll 2
+  for (int i = threadIdx.x * V; i < W; i += blockDim.x * V) {
+    float e[V], wv[V];
+    if constexpr (V == 4) {
+      load4(er + i, e);
+      load4(w + i, wv);
+#pragma unroll
+      for (int k = 0; k < V; ++k) e[k] *= inv * wv[k];
+      store4(h + row * (long)W + i, e);
+    } else {
+      stf(h + row * (long)W + i, ldf(er + i) * inv * w[i]);
+    }
+  }
 }
 
 std::vector<at::Tensor> streams_start(at::Tensor table, at::Tensor tokens, int64_t streams, at::Tensor w_in,
@@ -222,11 +241,18 @@ std::vector<at::Tensor> streams_start(at::Tensor table, at::Tensor tokens, int64
   TORCH_CHECK(S >= 1 && S <= 32 && wi.is_cuda() && wi.numel() == S && w.is_cuda() && w.numel() == W);
   at::Tensor x = at::empty({N, S, W}, table.options().dtype(at::kFloat));
   at::Tensor h = at::empty({N, W}, table.options());
+  auto al16 = [](const at::Tensor& t) { return reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0; };
+  const bool vec = W % 4 == 0 && al16(table) && al16(w) && al16(x) && al16(h);
   if (N > 0) {
     SERVING_DISPATCH_ACT(table, TE, {
-      hipLaunchKernelGGL(streams_start_kernel<TE>, dim3((unsigned)N), dim3(256), 0, stream(), ptr<TE>(h),
-                         x.data_ptr<float>(), ptr<TE>(table), (const long*)tokens.data_ptr<int64_t>(),
-                         wi.data_ptr<float>(), w.data_ptr<float>(), W, S, (float)eps);
+      if (vec)
+        hipLaunchKernelGGL((streams_start_kernel<TE, 4>), dim3((unsigned)N), dim3(256), 0, stream(), ptr<TE>(h),
+                           x.data_ptr<float>(), ptr<TE>(table), (const long*)tokens.data_ptr<int64_t>(),
+                           wi.data_ptr<float>(), w.data_ptr<float>(), W, S, (float)eps);
+      else
+        hipLaunchKernelGGL((streams_start_kernel<TE, 1>), dim3((unsigned)N), dim3(256), 0, stream(), ptr<TE>(h),
+                           x.data_ptr<float>(), ptr<TE>(table), (const long*)tokens.data_ptr<int64_t>(),
+                           wi.data_ptr<float>(), w.data_ptr<float>(), W, S, (float)eps);
     });
     HIP_CHECK_LAST();
   }
