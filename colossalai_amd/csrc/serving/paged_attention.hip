@@ -3,8 +3,8 @@
 // soft cap on the scaled score and an optional sink (one more place of score 0
 // in the softmax denominator that carries no value; with sink logits its score is learned per
 // head), an additive per-distance table, block summaries (one mean key/value per block of
-// positions that lies wholly before the window, kept in a small pool of their own; for
-// talking heads, every query head's weights applied to every key/value head's values), visibility
+// positions that lies wholly before the window, kept in a small pool of their own), for
+// talking heads every query head's weights applied to every key/value head's values, visibility
 // inside fixed blocks of positions instead of a window, a float32 factor per cached key (keys that
 // are normed when they are read), value heads shared by several key heads, and float32 output.
 //
@@ -17,6 +17,8 @@
 // the 64-key blocks. Phase 2: lane = value channel, the block's weights and
 // pool rows are broadcast from LDS. A prompt portion and a decode token run
 // the same code, so a position's result depends on nothing but the pages.
+// Calls without a distance table, block summaries or cross values run the form in row_attention.hip
+// where the row sizes fit it; bfloat16 prompt portions run the matrix-core kernel.
 #include "paged_attention.h"
 
 namespace cai {

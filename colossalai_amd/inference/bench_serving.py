@@ -118,8 +118,9 @@ def pooled_config(s: dict, experts: int = 32, top: int = 6, window: int = 1024, 
 
 def streams_config(s: dict, window: int = 1024, streams: int = 4) -> BekulixConfig:
     """As many layer runs as the size has layers, the first two looped twice: full attention over shared keys/values,
-    chunked differential attention (two maps of half the head size each over blocks of twice the ``window``: a query sees
-    as many keys on average) and windowed latent attention in turn, Llama's head sizes and feed-forward (ReLU), a latent of twice the head size."""
+    chunked differential attention (two maps of half the head size each over blocks of twice the ``window``, so that a
+    query sees as many keys on average) and windowed latent attention in turn; Llama's head sizes and feed-forward size
+    (ReLU), a latent of twice the head size."""
     W, H, G, D = s["width"], s["heads"], s["kv_heads"], s["dim"]
     att = dict(dim=D, heads=H, kv_heads=G, vdim=D, scale=D ** -0.5, q_temp=dict(coef=0.1, every=512))
     dif = dict(dim=D // 2, heads=H, kv_heads=G, vdim=D, scale=(D // 2) ** -0.5, diff=0.4, mask=dict(size=2 * window))
