@@ -14,7 +14,7 @@ void paged_kv_write(at::Tensor k, at::Tensor v, at::Tensor kpool, at::Tensor vpo
 at::Tensor grouped_rms_norm(at::Tensor x, at::Tensor weight, int64_t groups, double eps,
                             c10::optional<at::Tensor> residual, at::ScalarType out_dtype);
 at::Tensor head_rms_norm_gate(at::Tensor x, at::Tensor weight, double eps, c10::optional<at::Tensor> gate,
-                              at::ScalarType out_dtype);
+                              at::ScalarType out_dtype, int64_t gate_act);
 at::Tensor merge_rms_norm(at::Tensor a, at::Tensor wa, at::Tensor b, at::Tensor wb, double eps, at::Tensor out_w,
                           int64_t groups, at::Tensor residual);
 at::Tensor paged_attention(at::Tensor q, at::Tensor kpool, at::Tensor vpool, at::Tensor block_tables, at::Tensor cu,
@@ -64,6 +64,8 @@ c10::optional<at::Tensor> add_layer_norm(c10::optional<at::Tensor> residual, at:
                                          c10::optional<at::Tensor> w_out, double mult,
                                          c10::optional<at::Tensor> w_next, double eps, at::ScalarType out_dtype);
 void rotate_pairs(at::Tensor x, at::Tensor positions, at::Tensor freqs, at::Tensor out);
+void rotate_qk_write(at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor freqs, at::Tensor positions, at::Tensor kpool,
+                     at::Tensor vpool, at::Tensor rows);
 void latent_kv_write(at::Tensor dkv, at::Tensor norm_w, double eps, at::Tensor freqs, at::Tensor positions,
                      at::Tensor pool, at::Tensor rows);
 std::vector<at::Tensor> expert_sort(at::Tensor ids, int64_t num_experts);
@@ -80,7 +82,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("softcap", &s::softcap, "cap * tanh(x / cap), float32");
   m.def("paged_kv_write", &s::paged_kv_write, "scatter a ragged batch's keys/values into pool rows");
   m.def("grouped_rms_norm", &s::grouped_rms_norm, "grouped RMS norm, optional in-place residual add");
-  m.def("head_rms_norm_gate", &s::head_rms_norm_gate, "per-head RMS norm with shared weight and sigmoid gate");
+  m.def("head_rms_norm_gate", &s::head_rms_norm_gate, "per-head RMS norm with shared weight and sigmoid or silu gate");
   m.def("merge_rms_norm", &s::merge_rms_norm, "average of two RMS-normed branches, group norm, residual add");
   m.def("paged_attention", &s::paged_attention, "ragged paged attention: window, kept prefix, distance bias, gate, soft cap, sink");
   m.def("paged_attention_ext", &s::paged_attention_ext,
@@ -95,7 +97,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("silu_mul", &s::silu_mul, "silu(gate) * up of a packed [N, 2F] tensor");
   m.def("add_rms_norm", &s::add_rms_norm, "residual += a (+ b) in place, then the RMS norm of the sum");
   m.def("grouped_topk_route", &s::grouped_topk_route,
-        "sigmoid or softmax router: correction, group-limited top-k, renormalised or not");
+        "sigmoid, softmax or logits router: correction, group-limited top-k, renormalised, kept or softmax over the chosen");
   m.def("gelu_tanh_mul", &s::gelu_tanh_mul, "gelu_tanh(gate) * up of a packed [N, 2F] tensor");
   m.def("relu_mul", &s::relu_mul, "max(gate, 0) * up of a packed [N, 2F] tensor");
   m.def("query_norm_key_write", &s::query_norm_key_write,
@@ -107,6 +109,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("add_layer_norm", &s::add_layer_norm,
         "residual += mult * layer_norm(y) * w_out in place, then the layer norm of the sum (weight, no bias)");
   m.def("rotate_pairs", &s::rotate_pairs, "rotary positions on neighbouring pairs, strided in and out");
+  m.def("rotate_qk_write", &s::rotate_qk_write,
+        "rotary positions on neighbouring pairs: queries in place, keys into pool rows, values into pool rows");
   m.def("latent_kv_write", &s::latent_kv_write, "latent row: RMS norm + pair rotation + scatter into pool rows");
   m.def("expert_ffn_gemv", &s::expert_ffn_gemv, "chosen experts' feed-forward of a small step, matrix-vector kernels");
   m.def("expert_sort", &s::expert_sort, "stable sort of (token, expert) pairs by expert: offsets, source tokens, inverse");

@@ -258,6 +258,109 @@ void rotate_pairs(at::Tensor x, at::Tensor positions, at::Tensor freqs, at::Tens
   HIP_CHECK_LAST();
 }
 
+// ------------------------------------------- rotate queries and keys, write keys and values
+// One block per token: the sines and cosines of its half angles go to LDS once; then q [H, D] (row stride qs) is turned
+// in place and k [G, D] (ks), turned, and v [G, Dv] (vs) go to pool row rows[n]. VEC: eight channels per thread
+// (all sizes and strides multiples of 8, rows aligned); otherwise a pair of q or k, or a channel of v.
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void rotate_qk_write_kernel(
+    T* __restrict__ q, long qs, const T* __restrict__ k, long ks, const T* __restrict__ v, long vs,
+    const float* __restrict__ freqs, const int* __restrict__ positions, const int* __restrict__ rows,
+    T* __restrict__ kpool, T* __restrict__ vpool, int H, int G, int D, int Dv, int half) {
+  extern __shared__ float cs[];  // [2 * half]: cosine, sine per pair
+  const long n = blockIdx.x;
+  const float p = (float)positions[n];
+  for (int j = threadIdx.x; j < half; j += blockDim.x) sincosf(p * freqs[j], &cs[2 * j + 1], &cs[2 * j]);
+  __syncthreads();
+  T* qr = q + n * qs;
+  const T* kr = k + n * ks;
+  const T* vr = v + n * vs;
+  T* kd = kpool + (long)rows[n] * G * D;
+  T* vd = vpool + (long)rows[n] * G * Dv;
+  if constexpr (VEC) {
+    const int per = D / 8, nq = H * per, nk = G * per, nv = G * Dv / 8;
+    for (int i = threadIdx.x; i < nq + nk + nv; i += blockDim.x) {
+      float x[8];
+      if (i >= nq + nk) {
+        const int c = 8 * (i - nq - nk);
+        load8(vr + c, x);
+        store8(vd + c, x);
+        continue;
+      }
+      const bool isq = i < nq;
+      const int u = isq ? i : i - nq;
+      const int pair = 4 * (u % per);          // first pair of these channels inside its head
+      load8((isq ? qr : kr) + 8 * u, x);
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (pair + e < half) {
+          const float c = cs[2 * (pair + e)], s = cs[2 * (pair + e) + 1], a = x[2 * e], b = x[2 * e + 1];
+          x[2 * e] = a * c - b * s;
+          x[2 * e + 1] = b * c + a * s;
+        }
+      store8((isq ? qr : kd) + 8 * u, x);
+    }
+  } else {
+    const int per = (D + 1) / 2, nq = H * per, nk = G * per, nv = G * Dv;
+    for (int i = threadIdx.x; i < nq + nk + nv; i += blockDim.x) {
+      if (i >= nq + nk) {
+        const int c = i - nq - nk;
+        vd[c] = vr[c];
+        continue;
+      }
+      const bool isq = i < nq;
+      const int u = isq ? i : i - nq;
+      const int pair = u % per;
+      const long at = (long)(u / per) * D + 2 * pair;
+      const T* src = isq ? qr : kr;
+      T* dst = isq ? qr : kd;
+      const float a = ldf(src + at);
+      if (2 * pair + 1 >= D) {
+        stf(dst + at, a);
+        continue;
+      }
+      const float b = ldf(src + at + 1);
+      const float c = pair < half ? cs[2 * pair] : 1.0f, s = pair < half ? cs[2 * pair + 1] : 0.0f;
+      stf(dst + at, a * c - b * s);
+      stf(dst + at + 1, b * c + a * s);
+    }
+  }
+}
+
+void rotate_qk_write(at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor freqs, at::Tensor positions, at::Tensor kpool,
+                     at::Tensor vpool, at::Tensor rows) {
+  check_act(q, "q"); check_act(k, "k"); check_act(v, "v");
+  TORCH_CHECK(q.dim() == 3 && k.dim() == 3 && v.dim() == 3 && kpool.dim() == 4 && vpool.dim() == 4);
+  const long N = q.size(0);
+  const int H = (int)q.size(1), D = (int)q.size(2), G = (int)k.size(1), Dv = (int)v.size(2);
+  TORCH_CHECK(k.size(0) == N && v.size(0) == N && k.size(2) == D && v.size(1) == G, "q/k/v sizes do not fit");
+  TORCH_CHECK(q.stride(2) == 1 && q.stride(1) == D && k.stride(2) == 1 && k.stride(1) == D && v.stride(2) == 1 &&
+              v.stride(1) == Dv, "q/k/v rows must be dense (row stride free)");
+  TORCH_CHECK(kpool.is_cuda() && vpool.is_cuda() && kpool.is_contiguous() && vpool.is_contiguous() &&
+              kpool.size(2) == G && kpool.size(3) == D && vpool.size(2) == G && vpool.size(3) == Dv &&
+              vpool.size(0) == kpool.size(0) && vpool.size(1) == kpool.size(1), "pools must be contiguous [pages, page, G, D]");
+  TORCH_CHECK(q.scalar_type() == k.scalar_type() && q.scalar_type() == v.scalar_type() &&
+              q.scalar_type() == kpool.scalar_type() && q.scalar_type() == vpool.scalar_type(),
+              "queries, keys, values and pools share one dtype");
+  check_i32(positions, "positions"); check_i32(rows, "rows");
+  TORCH_CHECK(positions.numel() == N && rows.numel() == N);
+  TORCH_CHECK(freqs.is_cuda() && is_f32(freqs) && freqs.is_contiguous() && 2 * freqs.numel() <= D && freqs.numel() <= 4096,
+              "freqs must be float32 [dims / 2] with dims <= D");
+  if (N == 0) return;
+  const int half = (int)freqs.numel();
+  SERVING_DISPATCH_ACT(q, T, {
+    const auto aligned = [](const at::Tensor& t) { return reinterpret_cast<uintptr_t>(t.data_ptr()) % (8 * sizeof(T)) == 0; };
+    const bool vec = D % 8 == 0 && Dv % 8 == 0 && q.stride(0) % 8 == 0 && k.stride(0) % 8 == 0 && v.stride(0) % 8 == 0 &&
+                     aligned(q) && aligned(k) && aligned(v) && aligned(kpool) && aligned(vpool);
+    auto kfn = vec ? rotate_qk_write_kernel<T, true> : rotate_qk_write_kernel<T, false>;
+    hipLaunchKernelGGL(kfn, dim3((unsigned)N), dim3(256), (size_t)2 * half * sizeof(float), stream(), ptr<T>(q),
+                       (long)q.stride(0), ptr<T>(k), (long)k.stride(0), ptr<T>(v), (long)v.stride(0),
+                       freqs.data_ptr<float>(), positions.data_ptr<int>(), rows.data_ptr<int>(), ptr<T>(kpool),
+                       ptr<T>(vpool), H, G, D, Dv, half);
+  });
+  HIP_CHECK_LAST();
+}
+
 // ------------------------------------------------------------- latent row write
 // One wave per token: dkv row [rank + R] (row-strided) -> pool row rows[n]: the first `rank`
 // channels RMS-normed with a weight (float32 statistics), the last R rotated pair-wise (the

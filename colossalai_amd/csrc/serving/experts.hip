@@ -1,6 +1,7 @@
 // Mixture-of-experts serving kernels:
 //   grouped_topk_route : sigmoid (or softmax) scores, a selection-only correction, group-limited
-//                        top-k with ties to the lower index, chosen scores renormalised (or kept);
+//                        top-k with ties to the lower index, chosen scores renormalised (or kept), or
+//                        choice by logits and softmax over the chosen ones;
 //   expert_ffn_gemv    : a small step's chosen experts as two matrix-vector kernels
 //                        (up + squared ReLU per (token, expert) pair, then the weighted
 //                        down products of a token summed with its base row) — only the
@@ -21,7 +22,7 @@ namespace serving {
 __global__ __launch_bounds__(256) void grouped_topk_route_kernel(
     int* __restrict__ ids, float* __restrict__ wts, const float* __restrict__ logits, long ld,
     const float* __restrict__ corr, long N, int E, int top, int groups, int keep, int group_top, float eps,
-    int softmax, int renorm) {
+    int score_fn, int renorm) {
   extern __shared__ float lds[];
   const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
   float* sc = lds + (long)wid * (2 * E + groups + top);
@@ -31,7 +32,7 @@ __global__ __launch_bounds__(256) void grouped_topk_route_kernel(
   const long tok = (long)blockIdx.x * 4 + wid;
   const bool live = tok < N;
   const long n = live ? tok : N - 1;
-  if (softmax) {  // over all experts, float32: exp(z - max) / sum
+  if (score_fn == 1) {  // softmax over all experts, float32: exp(z - max) / sum
     float mx = -INFINITY;
     for (int e = lane; e < E; e += 64) mx = fmaxf(mx, logits[n * ld + e]);
     mx = wave_reduce_max(mx);
@@ -49,7 +50,7 @@ __global__ __launch_bounds__(256) void grouped_topk_route_kernel(
     }
   } else {
     for (int e = lane; e < E; e += 64) {
-      const float s = sigmoidf_(logits[n * ld + e]);
+      const float z = logits[n * ld + e], s = score_fn == 2 ? z : sigmoidf_(z);
       sc[e] = s;
       ch[e] = s + (corr != nullptr ? corr[e] : 0.0f);
     }
@@ -109,6 +110,14 @@ __global__ __launch_bounds__(256) void grouped_topk_route_kernel(
     total += sc[bi];
     __syncthreads();
   }
+  if (score_fn == 2) {  // softmax over the chosen logits
+    float mx = -INFINITY, sum = 0.0f;
+    for (int t = 0; t < top; ++t) mx = fmaxf(mx, pick[t]);
+    for (int t = 0; t < top; ++t) sum += expf(pick[t] - mx);
+    if (live)
+      for (int t = lane; t < top; t += 64) wts[tok * top + t] = expf(pick[t] - mx) / sum;
+    return;
+  }
   if (live)
     for (int t = lane; t < top; t += 64) wts[tok * top + t] = renorm ? pick[t] / (total + eps) : pick[t];
 }
@@ -118,7 +127,7 @@ std::vector<at::Tensor> grouped_topk_route(at::Tensor logits, c10::optional<at::
                                            double renorm_eps, int64_t score_fn, bool renorm) {
   TORCH_CHECK(logits.is_cuda() && is_f32(logits) && logits.dim() == 2 && logits.stride(1) == 1,
               "router logits must be float32 [N, E] with unit inner stride");
-  TORCH_CHECK(score_fn == 0 || score_fn == 1, "score function: 0 = sigmoid, 1 = softmax");
+  TORCH_CHECK(score_fn >= 0 && score_fn <= 2, "score function: 0 = sigmoid, 1 = softmax, 2 = logits");
   const long N = logits.size(0);
   const int E = (int)logits.size(1);
   TORCH_CHECK(group_count >= 1 && E % group_count == 0 && group_keep >= 1 && group_keep <= group_count && group_top >= 1);

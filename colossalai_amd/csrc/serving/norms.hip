@@ -92,7 +92,7 @@ at::Tensor grouped_rms_norm(at::Tensor x, at::Tensor weight, int64_t groups, dou
 template <typename TI, typename TG, typename TO>
 __global__ __launch_bounds__(256) void head_rms_norm_gate_kernel(
     TO* __restrict__ out, const TI* __restrict__ x, long xs, const float* __restrict__ w, const TG* __restrict__ gate,
-    long gs, long units, int H, int D, float eps) {
+    long gs, long units, int H, int D, float eps, int silu) {
   const int lane = threadIdx.x & 63;
   const long unit = (long)blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
   if (unit >= units) return;
@@ -108,13 +108,17 @@ __global__ __launch_bounds__(256) void head_rms_norm_gate_kernel(
   const float inv = 1.0f / sqrtf(ssq / (float)D + eps);
   for (int i = lane; i < D; i += 64) {
     float y = ldf(xr + i) * inv * w[i];
-    if (gate != nullptr) y *= sigmoidf_(ldf(gate + n * gs + (long)h * D + i));
+    if (gate != nullptr) {
+      const float g = ldf(gate + n * gs + (long)h * D + i);
+      y *= silu ? g * sigmoidf_(g) : sigmoidf_(g);
+    }
     stf(out + (n * H + h) * (long)D + i, y);
   }
 }
 
 at::Tensor head_rms_norm_gate(at::Tensor x, at::Tensor weight, double eps, c10::optional<at::Tensor> gate,
-                              at::ScalarType out_dtype) {
+                              at::ScalarType out_dtype, int64_t gate_act) {
+  TORCH_CHECK(gate_act == 0 || gate_act == 1, "gate activation: 0 = sigmoid, 1 = silu");
   check_act(x, "x");
   TORCH_CHECK(x.dim() == 3 && x.stride(2) == 1 && x.stride(1) == x.size(2), "x must be [N, H, D] with dense rows");
   const long N = x.size(0);
@@ -137,12 +141,12 @@ at::Tensor head_rms_norm_gate(at::Tensor x, at::Tensor weight, double eps, c10::
         SERVING_DISPATCH_ACT(*gate, TG, {
           hipLaunchKernelGGL((head_rms_norm_gate_kernel<TI, TG, TO>), dim3(grid), dim3(256), 0, stream(), ptr<TO>(out),
                              ptr<TI>(x), (long)x.stride(0), w.data_ptr<float>(), ptr<TG>(*gate), gs, units, H, D,
-                             (float)eps);
+                             (float)eps, (int)gate_act);
         });
       } else {
         hipLaunchKernelGGL((head_rms_norm_gate_kernel<TI, float, TO>), dim3(grid), dim3(256), 0, stream(),
                            ptr<TO>(out), ptr<TI>(x), (long)x.stride(0), w.data_ptr<float>(), (const float*)nullptr,
-                           0L, units, H, D, (float)eps);
+                           0L, units, H, D, (float)eps, 0);
       }
     });
   });

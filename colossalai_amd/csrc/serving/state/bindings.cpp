@@ -29,7 +29,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   namespace s = cai::serving;
   m.def("short_conv", &s::short_conv, "short causal depthwise convolution with carried tail and optional bias");
   m.def("ssd_recurrence", &s::ssd_recurrence, "state-space recurrence with one decay per head, carried state");
-  m.def("gated_delta_rule", &s::gated_delta_rule, "gated delta rule with per-channel decay, carried state");
+  m.def("gated_delta_rule", &s::gated_delta_rule, "gated delta rule with a decay per key channel or per head, carried state");
   m.def("selective_scan", &s::selective_scan, "diagonal recurrence with a decay per channel, place and token, carried state");
   m.def("tied_gate_recurrence", &s::tied_gate_recurrence, "HGRN2-style recurrence, carried state");
 }

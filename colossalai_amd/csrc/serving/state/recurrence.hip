@@ -9,7 +9,8 @@
 // the start and the end of a portion: cutting a prompt differently cannot
 // change a result.
 //
-//   delta: S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q
+//   delta: S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q   (g per key channel, or one
+//          number per head and token)
 //   tied : S <- diag(f) S + (1 - f) v^T;                          o = S^T q
 //   ssd  : S <- a S + (dt v) k^T  (one decay a per head and token);   o = S^T q + D_skip v
 //
@@ -23,9 +24,10 @@ namespace serving {
 
 
 // ------------------------------------------------------------------ prologue
-// One block per token. q/k [N, G, D] row-strided; dt [N, H*D] row-strided.
+// One block per token. q/k [N, G, D] row-strided; dt [N, H*D] row-strided, or, HEAD, [N, H]: one decay per head; then
+// beta [N, H, 2] receives (beta, decay) and dec is unused.
 // T: type of q/k (the convolution's output), TL: type of the gate and decay logits (projections).
-template <typename T, typename TL>
+template <typename T, typename TL, bool HEAD>
 __global__ __launch_bounds__(256) void delta_prepare_kernel(
     float* __restrict__ qn, float* __restrict__ kn, float* __restrict__ dec, float* __restrict__ beta,
     const T* __restrict__ q, long qs, const T* __restrict__ k, long ks, const TL* __restrict__ bl, long bs,
@@ -47,12 +49,19 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(
     float* dst = (isq ? qn : kn) + (n * G + g) * (long)D;
     for (int i = lane; i < D; i += 64) dst[i] = ldf(src + i) * inv;
   }
-  const int HD = H * D;
-  for (int i = threadIdx.x; i < HD; i += blockDim.x) {
-    const float a = expf(A_log[i / D]);
-    dec[n * HD + i] = expf(-a * softplusf_(ldf(dt + n * ds + i) + dt_bias[i]));
+  if constexpr (HEAD) {
+    for (int h = threadIdx.x; h < H; h += blockDim.x) {
+      beta[2 * (n * H + h)] = sigmoidf_(ldf(bl + n * bs + h));
+      beta[2 * (n * H + h) + 1] = expf(-expf(A_log[h]) * softplusf_(ldf(dt + n * ds + h) + dt_bias[h]));
+    }
+  } else {
+    const int HD = H * D;
+    for (int i = threadIdx.x; i < HD; i += blockDim.x) {
+      const float a = expf(A_log[i / D]);
+      dec[n * HD + i] = expf(-a * softplusf_(ldf(dt + n * ds + i) + dt_bias[i]));
+    }
+    for (int h = threadIdx.x; h < H; h += blockDim.x) beta[n * H + h] = sigmoidf_(ldf(bl + n * bs + h));
   }
-  for (int h = threadIdx.x; h < H; h += blockDim.x) beta[n * H + h] = sigmoidf_(ldf(bl + n * bs + h));
 }
 
 template <typename T>
@@ -109,10 +118,11 @@ DEV_INLINE float reduce_p(float v) {
 // prompt (D = 128): NC = 2 is 1.5x slower per layer than NC = 1 - a single long sequence is
 // bound by the instructions a wave issues per token, not by latencies that a second chain could
 // hide - so NC stays 1.
-// MODE: 0 = tied, 1 = delta, 2 = ssd. In ssd mode the operand rows are q and k (no per-channel gate) with the
+// MODE: 0 = tied, 1 = delta, 2 = ssd, 3 = delta with one decay per head and token. In ssd mode the operand rows are q and k (no per-channel gate) with the
 // token stride qk_ts, `beta` holds two scalars per (token, head), the decay a and the step dt, and `skip` [H] the
-// weight of the direct path.
-constexpr int SCAN_TIED = 0, SCAN_DELTA = 1, SCAN_SSD = 2;
+// weight of the direct path. Mode 3 takes its operands like ssd (q, k; `beta` holds beta and the decay) and applies the
+// decay to the dot product S^T k instead of ahead of it, so the state is read once and written once per token.
+constexpr int SCAN_TIED = 0, SCAN_DELTA = 1, SCAN_SSD = 2, SCAN_DELTA_HEAD = 3;
 
 template <int P, int DPL, int MODE, typename TV>
 __global__ __launch_bounds__(256) void matrix_state_scan_kernel(
@@ -120,11 +130,12 @@ __global__ __launch_bounds__(256) void matrix_state_scan_kernel(
     const float* __restrict__ beta, const TV* __restrict__ v, long vs, float* __restrict__ state, long ss,
     const int* __restrict__ cu, const int* __restrict__ start, const int* __restrict__ slots, int H, int rep, int D,
     int Dv, long qk_ts, int vec_ok, const float* __restrict__ skip) {
-  constexpr bool DELTA = MODE == SCAN_DELTA, SSD = MODE == SCAN_SSD;
+  constexpr bool DELTA = MODE == SCAN_DELTA, DHEAD = MODE == SCAN_DELTA_HEAD, SSD = MODE == SCAN_SSD;
+  constexpr bool PAIR = SSD || DHEAD;         // operands q, k and two scalars per (token, head)
   constexpr int Dp = P * DPL;                 // padded key size
   constexpr int CT = Dp > 128 ? 8 : 16;       // tokens per staged chunk
   constexpr int NOPS = DELTA ? 3 : 2;         // q, (k,) gate; ssd: q, k
-  constexpr int NB = SSD ? 2 : 1;             // scalars per (token, head)
+  constexpr int NB = PAIR ? 2 : 1;            // scalars per (token, head)
   constexpr int NC = 1;                       // value channels per lane
   constexpr int CPW = 4 * 64 / P;             // lanes groups (one channel each) per block
   constexpr int CPB = CPW * NC;               // value channels per block
@@ -165,9 +176,9 @@ __global__ __launch_bounds__(256) void matrix_state_scan_kernel(
   float r_v[R_V], r_b = 0.0f;
   const bool rows_vec = (D % 4) == 0 && vec_ok;
   const float* q_head = q + (long)hq * D;
-  const float* k_head = (DELTA || SSD) ? k + (long)hq * D : nullptr;
-  const float* g_head = SSD ? nullptr : gate + (long)h * D;
-  const long qk_stride = SSD ? qk_ts : (long)Hq * D, g_stride = (long)H * D;
+  const float* k_head = (DELTA || PAIR) ? k + (long)hq * D : nullptr;
+  const float* g_head = PAIR ? nullptr : gate + (long)h * D;
+  const long qk_stride = PAIR ? qk_ts : (long)Hq * D, g_stride = (long)H * D;
   const float dskip = SSD ? skip[h] : 0.0f;
   auto fetch = [&](int tb) {  // chunk starting at token tb -> registers
 #pragma unroll
@@ -176,7 +187,7 @@ __global__ __launch_bounds__(256) void matrix_state_scan_kernel(
       const int rowi = i / RF4, f4 = i % RF4;
       const int tok = rowi / NOPS, op = rowi % NOPS;
       const int t = tb + tok, d = f4 * 4;
-      const bool is_gate = !SSD && op == NOPS - 1;
+      const bool is_gate = !PAIR && op == NOPS - 1;
       const float fill = is_gate ? 1.0f : 0.0f;
       float4v val = {fill, fill, fill, fill};
       if (i < OPF4 && t < t1 && d < D) {
@@ -199,7 +210,7 @@ __global__ __launch_bounds__(256) void matrix_state_scan_kernel(
       r_v[r] = (i < CT * CPB && t < t1) ? ldf(v + (long)t * vs + (long)h * Dv + ch) : 0.0f;
     }
     if (DELTA) r_b = (tid < CT && tb + tid < t1) ? beta[(long)(tb + tid) * H + h] : 0.0f;
-    if (SSD) r_b = (tid < 2 * CT && tb + tid / 2 < t1) ? beta[((long)(tb + tid / 2) * H + h) * 2 + (tid & 1)] : 0.0f;
+    if (PAIR) r_b = (tid < 2 * CT && tb + tid / 2 < t1) ? beta[((long)(tb + tid / 2) * H + h) * 2 + (tid & 1)] : 0.0f;
   };
   auto stash = [&](int buf) {  // registers -> LDS buffer ([CT][NOPS][Dp], the order the rows were fetched in)
 #pragma unroll
@@ -212,7 +223,7 @@ __global__ __launch_bounds__(256) void matrix_state_scan_kernel(
       const int i = tid + 256 * r;
       if (i < CT * CPB) v_buf[buf * CT * CPB + i] = r_v[r];
     }
-    if ((DELTA || SSD) && tid < NB * CT) b_buf[buf * NB * CT + tid] = r_b;
+    if ((DELTA || PAIR) && tid < NB * CT) b_buf[buf * NB * CT + tid] = r_b;
   };
 
   fetch(t0);
@@ -230,17 +241,17 @@ __global__ __launch_bounds__(256) void matrix_state_scan_kernel(
       for (int j = 0; j < DPL; j += 4) {
         const float4v a = *reinterpret_cast<const float4v*>(row + j);
         qc[j] = a[0]; qc[j + 1] = a[1]; qc[j + 2] = a[2]; qc[j + 3] = a[3];
-        if (DELTA || SSD) {
+        if (DELTA || PAIR) {
           const float4v kk = *reinterpret_cast<const float4v*>(row + Dp + j);
           kc[j] = kk[0]; kc[j + 1] = kk[1]; kc[j + 2] = kk[2]; kc[j + 3] = kk[3];
         }
-        if (!SSD) {
+        if (!PAIR) {
           const float4v gg = *reinterpret_cast<const float4v*>(row + (NOPS - 1) * Dp + j);
           gc[j] = gg[0]; gc[j + 1] = gg[1]; gc[j + 2] = gg[2]; gc[j + 3] = gg[3];
         }
       }
-      const float bc = (DELTA || SSD) ? b_buf[(buf * CT + tt) * NB] : 0.0f;         // delta: beta; ssd: the decay a
-      const float dtc = SSD ? b_buf[(buf * CT + tt) * NB + 1] : 0.0f;               // ssd: the step dt
+      const float bc = (DELTA || PAIR) ? b_buf[(buf * CT + tt) * NB] : 0.0f;        // delta: beta; ssd: the decay a
+      const float dtc = PAIR ? b_buf[(buf * CT + tt) * NB + 1] : 0.0f;              // ssd: the step dt; delta: the decay
 #pragma unroll
       for (int x = 0; x < NC; ++x) {
         const float vc = v_buf[buf * CT * CPB + tt * CPB + x * CPW + cl];
@@ -260,6 +271,21 @@ __global__ __launch_bounds__(256) void matrix_state_scan_kernel(
           for (int j = 0; j < DPL; j += 2) {
             S[x][j] += kc[j] * u;
             S[x][j + 1] += kc[j + 1] * u;
+            oa += S[x][j] * qc[j];
+            ob += S[x][j + 1] * qc[j + 1];
+          }
+        } else if (DHEAD) {
+          float da = 0.0f, db = 0.0f;
+#pragma unroll
+          for (int j = 0; j < DPL; j += 2) {
+            da += S[x][j] * kc[j];
+            db += S[x][j + 1] * kc[j + 1];
+          }
+          const float u = bc * (vc - dtc * reduce_p<P>(da + db));
+#pragma unroll
+          for (int j = 0; j < DPL; j += 2) {
+            S[x][j] = dtc * S[x][j] + kc[j] * u;
+            S[x][j + 1] = dtc * S[x][j + 1] + kc[j + 1] * u;
             oa += S[x][j] * qc[j];
             ob += S[x][j + 1] * qc[j + 1];
           }
@@ -307,7 +333,8 @@ static void launch_scan(float* out, const float* q, const float* k, const float*
   // A step of single tokens (decoding) is all state traffic: a lane then holds 32 rows of its channel, so that few
   // lanes share a channel, a wave's loads of one state row cover 16 to 64 neighbouring channels and a block 64 to
   // 256 (whole cache lines), instead of 4 channels per wave when 16 lanes split a channel of 128 rows.
-  const bool wide = MODE == SCAN_SSD && short_step;
+  constexpr bool PAIR = MODE == SCAN_SSD || MODE == SCAN_DELTA_HEAD;
+  const bool wide = PAIR && short_step;
   const int dpl = wide ? 32 : D > 128 ? 16 : 8;
   int P = 1;
   while (P * dpl < D) P <<= 1;
@@ -317,7 +344,7 @@ static void launch_scan(float* out, const float* q, const float* k, const float*
 #define SCAN_CASE(PP, DD)                                                                                          \
   hipLaunchKernelGGL((matrix_state_scan_kernel<PP, DD, MODE, TV>), grid, dim3(256), smem, stream(), out, q, k,    \
                      gate, beta, v, vs, state, ss, cu, start, slots, H, rep, D, Dv, qk_ts, vec_ok, skip)
-  if constexpr (MODE == SCAN_SSD) {
+  if constexpr (PAIR) {
     if (wide) {
       if (P == 1) SCAN_CASE(1, 32);
       else if (P == 2) SCAN_CASE(2, 32);
@@ -357,29 +384,39 @@ at::Tensor gated_delta_rule(at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor
   const int G = (int)q.size(1), D = (int)q.size(2), H = (int)v.size(1), Dv = (int)v.size(2);
   TORCH_CHECK(k.size(0) == N && v.size(0) == N && k.size(1) == G && k.size(2) == D && H % G == 0);
   TORCH_CHECK(beta_logit.dim() == 2 && beta_logit.size(0) == N && beta_logit.size(1) == H && beta_logit.stride(1) == 1);
-  TORCH_CHECK(dt.dim() == 2 && dt.size(0) == N && dt.size(1) == (long)H * D && dt.stride(1) == 1);
+  TORCH_CHECK(dt.dim() == 2 && dt.size(0) == N && dt.stride(1) == 1 && (dt.size(1) == H || dt.size(1) == (long)H * D),
+              "dt must be [N, H] (a decay per head) or [N, H * D] (per key channel)");
   TORCH_CHECK(q.scalar_type() == k.scalar_type() && q.scalar_type() == v.scalar_type() &&
               beta_logit.scalar_type() == dt.scalar_type(), "q/k/v share one dtype, the logits another or the same");
   check_state(state, H, D, Dv);
   check_i32(cu, "cu"); check_i32(start, "start"); check_i32(slots, "slots");
   const int B = (int)start.numel();
+  const bool head = dt.size(1) == H;
   at::Tensor Af = f32c(A_log), bf = f32c(dt_bias);
-  TORCH_CHECK(Af.numel() == H && bf.numel() == (long)H * D);
+  TORCH_CHECK(Af.numel() == H && bf.numel() == dt.size(1) && Af.is_cuda() && bf.is_cuda());
   auto fo = q.options().dtype(at::kFloat);
   at::Tensor out = at::empty({N, H, Dv}, fo);
   if (N == 0) return out;
-  at::Tensor qn = at::empty({N, G, D}, fo), kn = at::empty({N, G, D}, fo), dec = at::empty({N, H, D}, fo),
-             beta = at::empty({N, H}, fo);
+  at::Tensor qn = at::empty({N, G, D}, fo), kn = at::empty({N, G, D}, fo), dec, beta = at::empty({N, H, head ? 2 : 1}, fo);
+  if (!head) dec = at::empty({N, H, D}, fo);
+  float* decp = head ? nullptr : dec.data_ptr<float>();
   SERVING_DISPATCH_ACT(q, T, {
     SERVING_DISPATCH_ACT(dt, TL, {
-      hipLaunchKernelGGL((delta_prepare_kernel<T, TL>), dim3((unsigned)N), dim3(256), 0, stream(), qn.data_ptr<float>(),
-                         kn.data_ptr<float>(), dec.data_ptr<float>(), beta.data_ptr<float>(), ptr<T>(q),
+      auto kfn = head ? delta_prepare_kernel<T, TL, true> : delta_prepare_kernel<T, TL, false>;
+      hipLaunchKernelGGL(kfn, dim3((unsigned)N), dim3(256), 0, stream(), qn.data_ptr<float>(),
+                         kn.data_ptr<float>(), decp, beta.data_ptr<float>(), ptr<T>(q),
                          (long)q.stride(0), ptr<T>(k), (long)k.stride(0), ptr<TL>(beta_logit),
                          (long)beta_logit.stride(0), ptr<TL>(dt), (long)dt.stride(0), Af.data_ptr<float>(),
                          bf.data_ptr<float>(), G, H, D, (float)unit_eps, (float)q_scale);
     });
     HIP_CHECK_LAST();
-    launch_scan<SCAN_DELTA, T>(out.data_ptr<float>(), qn.data_ptr<float>(), kn.data_ptr<float>(), dec.data_ptr<float>(),
+    if (head)
+      launch_scan<SCAN_DELTA_HEAD, T>(out.data_ptr<float>(), qn.data_ptr<float>(), kn.data_ptr<float>(), decp,
+                         beta.data_ptr<float>(), ptr<T>(v), (long)v.stride(0), state.data_ptr<float>(),
+                         (long)state.stride(0), cu.data_ptr<int>(), start.data_ptr<int>(), slots.data_ptr<int>(), B, H,
+                         H / G, D, Dv, (long)G * D, 1, nullptr, N <= 2L * B);
+    else
+      launch_scan<SCAN_DELTA, T>(out.data_ptr<float>(), qn.data_ptr<float>(), kn.data_ptr<float>(), decp,
                          beta.data_ptr<float>(), ptr<T>(v), (long)v.stride(0), state.data_ptr<float>(),
                          (long)state.stride(0), cu.data_ptr<int>(), start.data_ptr<int>(), slots.data_ptr<int>(), B, H,
                          H / G, D, Dv);

@@ -9,6 +9,7 @@ from .mubutar import MubutarConfig, MubutarForCausalLM
 from .vitinex import VitinexConfig, VitinexForCausalLM
 from .tarulix import TarulixConfig, TarulixForCausalLM
 from .bekulix import BekulixConfig, BekulixForCausalLM
+from .vosulorn import VosulornConfig, VosulornForCausalLM
 from .llama import LLAMA_CONFIGS, LlamaConfig, LlamaForCausalLM, llama_flops_per_token
 from .bert import BERT_CONFIGS, BertConfig, BertForMaskedLM, BertForSequenceClassification
 from .opt import OPT_CONFIGS, OPTConfig, OPTForCausalLM
@@ -23,7 +24,7 @@ from .whisper import WHISPER_CONFIGS, WhisperConfig, WhisperForConditionalGenera
 
 __all__ = ["load_pretrained", "model_class_for", "register_model", "registered_models",
            "KipiraxConfig", "KipiraxForCausalLM", "MubutarConfig", "MubutarForCausalLM", "VitinexConfig", "VitinexForCausalLM",
-           "TarulixConfig", "TarulixForCausalLM", "BekulixConfig", "BekulixForCausalLM",
+           "TarulixConfig", "TarulixForCausalLM", "BekulixConfig", "BekulixForCausalLM", "VosulornConfig", "VosulornForCausalLM",
            "LlamaConfig", "LlamaForCausalLM", "LLAMA_CONFIGS", "llama_flops_per_token",
            "OPTConfig", "OPTForCausalLM", "OPT_CONFIGS",
            "BertConfig", "BertForMaskedLM", "BertForSequenceClassification", "BERT_CONFIGS",

@@ -6,7 +6,7 @@ element-wise weight; with ``residual`` it adds the result to a float32 residual
 stream in place (norm on the sublayer's *output*). ``groups=1`` is plain RMS
 norm. ``head_rms_norm_gate`` normalises every head vector of a ``[N, H, D]``
 tensor with one shared ``[D]`` weight and optionally multiplies by
-``sigmoid(gate)``. ``add_rms_norm`` serves pre-norm layers: it adds one or two
+``sigmoid(gate)`` or ``silu(gate)``. ``add_rms_norm`` serves pre-norm layers: it adds one or two
 sublayer outputs to the float32 residual stream in place and hands back the
 RMS-normed stream for the next layer in one pass. ``gated_grouped_rms_norm``
 multiplies a row by ``silu(gate)`` *before* its grouped RMS norm (the output norm
@@ -50,19 +50,25 @@ def grouped_rms_norm(x, weight, groups: int, eps: float, residual: Optional[torc
     return grouped_rms_norm_ref(x, weight, groups, eps, residual, out_dtype)
 
 
-def head_rms_norm_gate_ref(x, weight, eps: float, gate=None, out_dtype=None):
+GATES = {"sigmoid": 0, "silu": 1}
+
+
+def head_rms_norm_gate_ref(x, weight, eps: float, gate=None, out_dtype=None, act: str = "sigmoid"):
     xf = x.float()
     y = xf * torch.rsqrt(xf.pow(2).mean(-1, keepdim=True) + eps) * weight.float()
     if gate is not None:
-        y = y * torch.sigmoid(gate.float().reshape(y.shape))
+        g = gate.float().reshape(y.shape)
+        y = y * (torch.sigmoid(g) if act == "sigmoid" else g * torch.sigmoid(g))
     return y.to(out_dtype or x.dtype)
 
 
-def head_rms_norm_gate(x, weight, eps: float, gate=None, out_dtype=None):
-    """x [N, H, D] (row-strided allowed), weight [D], gate logits [N, H * D] or None."""
+def head_rms_norm_gate(x, weight, eps: float, gate=None, out_dtype=None, act: str = "sigmoid"):
+    """x [N, H, D] (row-strided allowed), weight [D], gate [N, H * D] (what ``act``, "sigmoid" or "silu", is taken of)
+    or None."""
+    assert act in GATES
     if use_hip(x):
-        return serving_kernels().head_rms_norm_gate(x, weight, eps, gate, out_dtype or x.dtype)
-    return head_rms_norm_gate_ref(x, weight, eps, gate, out_dtype)
+        return serving_kernels().head_rms_norm_gate(x, weight, eps, gate, out_dtype or x.dtype, GATES[act])
+    return head_rms_norm_gate_ref(x, weight, eps, gate, out_dtype, act)
 
 
 def merge_rms_norm_ref(a, wa, b, wb, eps: float, out_w, groups: int, residual):

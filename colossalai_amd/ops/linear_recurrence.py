@@ -4,11 +4,12 @@ Every head keeps a float32 matrix ``S [D, Dv]`` per state slot (rows = key /
 query channels, columns = value channels) that is carried from step to step.
 Three update rules are provided:
 
-* ``gated_delta_rule`` — per-channel decay plus delta-rule write
+* ``gated_delta_rule`` — decay plus delta-rule write
   ``S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q``
-  with ``g = exp(-exp(A_log_h) * softplus(dt + dt_bias))`` per key channel,
-  ``beta = sigmoid(.)``, q and k scaled to unit length per head
-  (``x / sqrt(sum x^2 + unit_eps)``) and q further by ``q_scale``.
+  with ``g = exp(-exp(A_log_h) * softplus(dt + dt_bias))`` per key channel or one
+  number per head (the size of ``dt`` says which), ``beta = sigmoid(.)``, q and k
+  scaled to unit length per head (``x / sqrt(sum x^2 + unit_eps)``) and q further
+  by ``q_scale``.
 * ``tied_gate_recurrence`` (HGRN2) — the forget gate also sets the write:
   ``S <- diag(f) S + (1 - f) v^T;  o = S^T q`` with
   ``f = lower + (1 - lower) sigmoid(f_logit + f_bias)`` and ``q = silu(.)``.
@@ -53,8 +54,9 @@ def gated_delta_rule_ref(q, k, v, beta_logit, dt, A_log, dt_bias, state, batch: 
     kf = kf.repeat_interleave(rep, 1)
     vf = v.float()
     beta = torch.sigmoid(beta_logit.float())
+    # [N, H, D], or [N, H, 1] for one decay per head
     g = torch.exp(-torch.exp(A_log.float())[None, :, None]
-                  * F.softplus(dt.float().reshape(N, H, D) + dt_bias.float().reshape(H, D)))
+                  * F.softplus(dt.float().reshape(N, H, -1) + dt_bias.float().reshape(H, -1)))
     out = torch.empty(N, H, Dv, dtype=torch.float32, device=q.device)
 
     def step(S, t):
@@ -71,7 +73,8 @@ def gated_delta_rule_ref(q, k, v, beta_logit, dt, A_log, dt_bias, state, batch: 
 def gated_delta_rule(q, k, v, beta_logit, dt, A_log, dt_bias, state, batch: RaggedBatch,
                      unit_eps: float = 1e-6, q_scale: float = 1.0):
     """q, k [N, G, D]; v [N, H, Dv] (H a multiple of G; head h reads q/k head
-    h // (H / G)); beta_logit [N, H]; dt [N, H * D]; A_log [H]; dt_bias [H * D];
+    h // (H / G)); beta_logit [N, H]; dt [N, H * D] and dt_bias [H * D] (a decay per key
+    channel) or dt [N, H] and dt_bias [H] (one per head); A_log [H];
     state [slots, H, D, Dv] float32. Returns o [N, H, Dv] float32."""
     if use_hip(q):
         return serving_kernels().gated_delta_rule(q, k, v, beta_logit, dt, A_log, dt_bias, state, batch.cu,

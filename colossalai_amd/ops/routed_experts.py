@@ -15,7 +15,8 @@ weights:
 
 With ``score="softmax"`` the scores are the softmax of the logits over all
 experts, and with ``renorm=False`` the chosen scores are the mixing weights as
-they are.
+they are. With ``score="logits"`` the choice is made on the logits themselves and
+the mixing weights are the softmax over the chosen logits only.
 
 ``routed_expert_ffn`` runs ``down_e(act(up_e(h)))`` for each token's chosen
 experts and forms ``base + sum_j weight_j * y_j`` in float32. The activation is
@@ -54,7 +55,8 @@ GEMV_FALLBACK_PAIRS = 2048
 def grouped_topk_route_ref(logits, correction, top: int, group_count: int = 1, group_keep: int = 1,
                            group_top: int = 2, renorm_eps: float = 1e-20, score: str = "sigmoid", renorm: bool = True):
     N, E = logits.shape
-    s = torch.softmax(logits.float(), -1) if score == "softmax" else torch.sigmoid(logits.float())
+    z = logits.float()
+    s = torch.softmax(z, -1) if score == "softmax" else torch.sigmoid(z) if score == "sigmoid" else z
     choice = s + correction.float() if correction is not None else s
     if group_count > 1:
         per = E // group_count
@@ -67,17 +69,19 @@ def grouped_topk_route_ref(logits, correction, top: int, group_count: int = 1, g
         choice = grouped.masked_fill(~allowed[:, :, None], float("-inf")).reshape(N, E)
     idx = torch.sort(choice, dim=-1, descending=True, stable=True).indices[:, :top]
     w = s.gather(1, idx)
+    if score == "logits":
+        return idx.int(), torch.softmax(w, -1)
     return idx.int(), (w / (w.sum(-1, keepdim=True) + renorm_eps) if renorm else w)
 
 
-SCORES = {"sigmoid": 0, "softmax": 1}
+SCORES = {"sigmoid": 0, "softmax": 1, "logits": 2}
 
 
 def grouped_topk_route(logits, correction, top: int, group_count: int = 1, group_keep: int = 1,
                        group_top: int = 2, renorm_eps: float = 1e-20, score: str = "sigmoid", renorm: bool = True):
     """logits [N, E] float32 (rows may be strided), correction [E] or None -> (ids [N, top] int32, weights
-    [N, top] float32). ``score``: "sigmoid" or "softmax" (over all experts); ``renorm``: divide the chosen scores
-    by their sum."""
+    [N, top] float32). ``score``: "sigmoid", "softmax" (over all experts) or "logits" (weights: softmax over the
+    chosen); ``renorm``: divide the chosen scores by their sum."""
     N, E = logits.shape
     assert score in SCORES
     assert E % group_count == 0 and 0 < group_keep <= group_count
