@@ -30,12 +30,13 @@ def parse_args():
     p.add_argument("--steps", type=int, default=5)
     p.add_argument("--warmup", type=int, default=2)
     p.add_argument("--workload", type=str, default="train", choices=["train", "serve-hybrid", "serve-moe", "serve-latent", "serve-pooled",
-                                                                       "serve-streams"],
+                                                                       "serve-streams", "serve-delta"],
                    help="train: the headline training step (default). serve-hybrid / serve-moe / serve-latent / "
-                        "serve-pooled / serve-streams: prefill/decode tokens/s of the Kipirax hybrid / the Mubutar routed-experts model / "
+                        "serve-pooled / serve-streams / serve-delta: prefill/decode tokens/s of the Kipirax hybrid / the Mubutar routed-experts model / "
                         "the Vitinex latent-attention + state-space model / the Tarulix window + block-summary + "
-                        "selective-scan model / the Bekulix multi-stream model next to a Llama of equal size (the last three "
-                        "also next to Mubutar, the last also next to Vitinex), all "
+                        "selective-scan model / the Bekulix multi-stream model / the Vosulorn latent-attention + delta-rule "
+                        "model next to a Llama of equal size (the last four also next to Mubutar, the last two also "
+                        "next to Vitinex, the last also next to Kipirax), all "
                         "through the continuous-batching engine")
     p.add_argument("--serve-sizes", type=str, default="w2048,w4096")
     p.add_argument("--model", type=str, default="llama-7b")
@@ -72,7 +73,7 @@ def serve_comparison(args, kind):
 
 def main():
     args = parse_args()
-    if args.workload in ("serve-hybrid", "serve-moe", "serve-latent", "serve-pooled", "serve-streams"):
+    if args.workload in ("serve-hybrid", "serve-moe", "serve-latent", "serve-pooled", "serve-streams", "serve-delta"):
         return serve_comparison(args, args.workload.split("-")[1])
     import colossalai_amd
     from colossalai_amd.models import LLAMA_CONFIGS, LlamaForCausalLM, llama_flops_per_token

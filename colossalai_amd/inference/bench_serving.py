@@ -1,15 +1,17 @@
 """Serving throughput of the ragged-step models next to a Llama of equal width,
 depth and per-token work, all through ``ContinuousBatchEngine``: prefill tokens/s
 of one long prompt and decode tokens/s of a batch of running sequences. Random
-weights, synthetic tokens. Five comparisons: the Kipirax hybrid (paged window
+weights, synthetic tokens. Six comparisons: the Kipirax hybrid (paged window
 attention + recurrent state), Mubutar (sink-softmax attention with shared
 keys, routed experts), Vitinex (latent attention + state-space layers in a
 looped block, routed experts), Tarulix (windowed attention with a distance
 table and a learned sink; window + block summaries + talking heads beside a
-selective scan; gated experts with identity experts) and Bekulix (parallel residual
+selective scan; gated experts with identity experts), Bekulix (parallel residual
 streams; attention whose values are its keys, chunked differential attention and
-windowed latent attention; looped block), the last three also next to Mubutar, whose
-kernels are the closest, and Bekulix also next to Vitinex.
+windowed latent attention; looped block) and Vosulorn (latent attention with shared
+latents, chunked rotary attention with a learned sink, per-head gated delta rule,
+gated experts), the last four also next to Mubutar, Bekulix and Vosulorn also next
+to Vitinex, and Vosulorn also next to Kipirax.
 """
 
 import json
@@ -19,12 +21,13 @@ from typing import Dict, List
 import torch
 
 from ..models import (BekulixConfig, BekulixForCausalLM, KipiraxConfig, KipiraxForCausalLM, LlamaConfig, LlamaForCausalLM, MubutarConfig,
-                      MubutarForCausalLM, TarulixConfig, TarulixForCausalLM, VitinexConfig, VitinexForCausalLM)
+                      MubutarForCausalLM, TarulixConfig, TarulixForCausalLM, VitinexConfig, VitinexForCausalLM, VosulornConfig,
+                      VosulornForCausalLM)
 from .config import InferenceConfig
 from .paged_engine import ContinuousBatchEngine
 
 __all__ = ["SIZES", "hybrid_config", "llama_config", "moe_config", "latent_config", "pooled_config",
-           "streams_config",
+           "streams_config", "delta_config",
            "run_serving_comparison"]
 
 # width, layers, heads, kv_heads, head size, vocab
@@ -132,6 +135,23 @@ def streams_config(s: dict, window: int = 1024, streams: int = 4) -> BekulixConf
                          loop=dict(start=0, stop=2, times=2))
 
 
+def delta_config(s: dict, experts: int = 32, top: int = 6, chunk: int = 2048) -> VosulornConfig:
+    """Half the layers the gated delta rule (Kipirax's head sizes, two heads per query/key head), the others latent
+    attention (Vitinex's head and latent sizes; the second one reads the first one's latents) and chunked attention
+    (Llama's head sizes); with four layers one of the two delta layers makes room for the shared latents. Every layer
+    carries routed gated experts whose active matrices do the work of Llama's dense feed-forward."""
+    W, H, G, D = s["width"], s["heads"], s["kv_heads"], s["dim"]
+    lat = dict(dim=D // 2, rot_dim=D // 2, vdim=D, heads=H, kv_rank=2 * D, rot=dict(base=10000.0, dims=D // 2), scale=D ** -0.5)
+    att = dict(dim=D, heads=H, kv_heads=G, vdim=D, scale=D ** -0.5, mask=dict(size=chunk),
+               rot=dict(base=500000.0, dims=D, scaling=dict(factor=8.0, low=1.0, high=4.0, original=8192)))
+    delta = dict(conv=4, dim=D, heads=H, kv_heads=H // 2, vdim=D)
+    L, S, A, R = (("latent_attention", lat), ("latent_attention", dict(lat, kv_from=0)), ("attention", att), ("delta", delta))
+    kinds = [L, R, A, R, S, R, A, R] if s["layers"] >= 8 else [L, R, S, A]
+    mlp = dict(kind="moe", expert=dict(ff=_inter(W) // top // 32 * 32), router=dict(experts=experts, top=top))
+    layers = [dict(type=kinds[i % len(kinds)][0], mixer=kinds[i % len(kinds)][1], mlp=mlp) for i in range(s["layers"])]
+    return VosulornConfig(vocab=s["vocab"], width=W, layers=layers, norm_eps=1e-6, embedding_scale=W ** 0.5)
+
+
 def llama_config(s: dict, max_positions: int) -> LlamaConfig:
     # gate/up/down of 8/3 W carry the parameters of the hybrid's up/down of 4 W
     inter = _inter(s["width"])
@@ -222,6 +242,17 @@ def _streams_numbers(s: dict, prompt: int, batch: int, context: int, steps: int)
     return _ragged_numbers(model, cfg.vocab, prompt, batch, context, steps)
 
 
+def _delta_numbers(s: dict, prompt: int, batch: int, context: int, steps: int) -> Dict[str, float]:
+    cfg = delta_config(s)
+    model = VosulornForCausalLM(cfg).serving_dtype(torch.bfloat16).to("cuda").eval()
+    with torch.no_grad():
+        for p in model.parameters():
+            if p.dtype == torch.bfloat16:
+                p.normal_(0, 0.02)
+    model.prepare()
+    return _ragged_numbers(model, cfg.vocab, prompt, batch, context, steps)
+
+
 def _ragged_numbers(model, vocab: int, prompt: int, batch: int, context: int, steps: int) -> Dict[str, float]:
     page = 64
     blocks = max(prompt, batch * (context + steps + page)) // page + batch + 2
@@ -277,18 +308,21 @@ def _llama_numbers(s: dict, prompt: int, batch: int, context: int, steps: int) -
 
 def run_serving_comparison(sizes: List[str], prompt: int = 4096, batch: int = 16, context: int = 1024,
                            steps: int = 32, kind: str = "hybrid") -> dict:
-    """``kind``: "hybrid" (Kipirax), "moe" (Mubutar), "latent" (Vitinex), "pooled" (Tarulix) or "streams" (Bekulix),
-    each next to Llama; the last three also next to Mubutar, "streams" also next to Vitinex."""
+    """``kind``: "hybrid" (Kipirax), "moe" (Mubutar), "latent" (Vitinex), "pooled" (Tarulix), "streams" (Bekulix) or
+    "delta" (Vosulorn), each next to Llama; the last four also next to Mubutar, "streams" and "delta" also next to
+    Vitinex, "delta" also next to Kipirax."""
     ours = {"hybrid": _hybrid_numbers, "moe": _moe_numbers, "latent": _latent_numbers, "pooled": _pooled_numbers,
-            "streams": _streams_numbers}[kind]
+            "streams": _streams_numbers, "delta": _delta_numbers}[kind]
     out = {}
     for name in sizes:
         s = SIZES[name]
         out[name] = {kind: ours(s, prompt, batch, context, steps)}
-        if kind in ("latent", "pooled", "streams"):
+        if kind in ("latent", "pooled", "streams", "delta"):
             out[name]["moe"] = _moe_numbers(s, prompt, batch, context, steps)
-        if kind == "streams":
+        if kind in ("streams", "delta"):
             out[name]["latent"] = _latent_numbers(s, prompt, batch, context, steps)
+        if kind == "delta":
+            out[name]["hybrid"] = _hybrid_numbers(s, prompt, batch, context, steps)
         out[name]["llama"] = _llama_numbers(s, prompt, batch, context, steps)
         out[name]["shape"] = dict(s, prompt=prompt, batch=batch, context=context)
     return out
