@@ -14,7 +14,12 @@ at::Tensor ssd_recurrence(at::Tensor x, at::Tensor Bm, at::Tensor Cm, at::Tensor
                           at::Tensor slots);
 at::Tensor gated_delta_rule(at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor beta_logit, at::Tensor dt,
                             at::Tensor A_log, at::Tensor dt_bias, at::Tensor state, at::Tensor cu, at::Tensor start,
-                            at::Tensor slots, double unit_eps, double q_scale);
+                            at::Tensor slots, double unit_eps, double q_scale, c10::optional<at::Tensor> chunks,
+                            c10::optional<at::Tensor> seq_chunks);
+at::Tensor conv_delta_rule(at::Tensor x, at::Tensor taps, c10::optional<at::Tensor> tail, at::Tensor beta_logit, at::Tensor dt,
+                           at::Tensor A_log, at::Tensor dt_bias, at::Tensor state, at::Tensor cu, at::Tensor start,
+                           at::Tensor slots, at::Tensor tok_seq, int64_t groups, int64_t dim, double unit_eps, double q_scale,
+                           c10::optional<at::Tensor> chunks, c10::optional<at::Tensor> seq_chunks);
 at::Tensor tied_gate_recurrence(at::Tensor q, at::Tensor f_logit, at::Tensor v, at::Tensor f_bias, at::Tensor lower,
                                 at::Tensor state, at::Tensor cu, at::Tensor start, at::Tensor slots);
 at::Tensor selective_scan(at::Tensor x, at::Tensor dt_raw, at::Tensor A_log, at::Tensor Bm, at::Tensor Cm,
@@ -30,6 +35,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("short_conv", &s::short_conv, "short causal depthwise convolution with carried tail and optional bias");
   m.def("ssd_recurrence", &s::ssd_recurrence, "state-space recurrence with one decay per head, carried state");
   m.def("gated_delta_rule", &s::gated_delta_rule, "gated delta rule with a decay per key channel or per head, carried state");
+  m.def("conv_delta_rule", &s::conv_delta_rule,
+        "short convolution, unit-length q/k and gates in one launch, then the delta rule with a decay per head");
   m.def("selective_scan", &s::selective_scan, "diagonal recurrence with a decay per channel, place and token, carried state");
   m.def("tied_gate_recurrence", &s::tied_gate_recurrence, "HGRN2-style recurrence, carried state");
 }

@@ -17,7 +17,7 @@
 // A prologue kernel turns the raw projections into float32 operands once per
 // token (unit-length q/k, decay from its logits, gates), so the sequential
 // loop holds no transcendental.
-#include "../serving_common.h"
+#include "delta.h"
 
 namespace cai {
 namespace serving {
@@ -25,14 +25,14 @@ namespace serving {
 
 // ------------------------------------------------------------------ prologue
 // One block per token. q/k [N, G, D] row-strided; dt [N, H*D] row-strided, or, HEAD, [N, H]: one decay per head; then
-// beta [N, H, 2] receives (beta, decay) and dec is unused.
+// beta [N, H, 2] receives (beta, decay), or (beta, log decay), and dec is unused.
 // T: type of q/k (the convolution's output), TL: type of the gate and decay logits (projections).
 template <typename T, typename TL, bool HEAD>
 __global__ __launch_bounds__(256) void delta_prepare_kernel(
     float* __restrict__ qn, float* __restrict__ kn, float* __restrict__ dec, float* __restrict__ beta,
     const T* __restrict__ q, long qs, const T* __restrict__ k, long ks, const TL* __restrict__ bl, long bs,
     const TL* __restrict__ dt, long ds, const float* __restrict__ A_log, const float* __restrict__ dt_bias, int G, int H,
-    int D, float unit_eps, float q_scale) {
+    int D, float unit_eps, float q_scale, int log_decay) {
   const long n = blockIdx.x;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, nw = blockDim.x >> 6;
   for (int u = wid; u < 2 * G; u += nw) {
@@ -52,7 +52,8 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(
   if constexpr (HEAD) {
     for (int h = threadIdx.x; h < H; h += blockDim.x) {
       beta[2 * (n * H + h)] = sigmoidf_(ldf(bl + n * bs + h));
-      beta[2 * (n * H + h) + 1] = expf(-expf(A_log[h]) * softplusf_(ldf(dt + n * ds + h) + dt_bias[h]));
+      const float lg = -expf(A_log[h]) * softplusf_(ldf(dt + n * ds + h) + dt_bias[h]);
+      beta[2 * (n * H + h) + 1] = log_decay ? lg : expf(lg);
     }
   } else {
     const int HD = H * D;
@@ -375,9 +376,23 @@ static void check_rows3(const at::Tensor& t, const char* name) {
   TORCH_CHECK(t.dim() == 3 && t.stride(2) == 1 && t.stride(1) == t.size(2), name, " must be [N, heads, dim] with dense rows");
 }
 
+void delta_head_scan(at::Tensor& out, const at::Tensor& q, const at::Tensor& k, const at::Tensor& gates, const at::Tensor& v,
+                     at::Tensor& state, const at::Tensor& cu, const at::Tensor& start, const at::Tensor& slots) {
+  const long N = q.size(0);
+  const int G = (int)q.size(1), D = (int)q.size(2), H = (int)v.size(1), Dv = (int)v.size(2), B = (int)start.numel();
+  SERVING_DISPATCH_ACT(v, T, {
+    launch_scan<SCAN_DELTA_HEAD, T>(out.data_ptr<float>(), q.data_ptr<float>(), k.data_ptr<float>(), (const float*)nullptr,
+                                    gates.data_ptr<float>(), ptr<T>(v), (long)v.stride(0), state.data_ptr<float>(),
+                                    (long)state.stride(0), cu.data_ptr<int>(), start.data_ptr<int>(), slots.data_ptr<int>(),
+                                    B, H, H / G, D, Dv, (long)G * D, 1, nullptr, N <= 2L * B);
+  });
+}
+
+// With one decay per head, `chunks` and `seq_chunks` (RaggedBatch.chunk_tables) ask for the chunked form.
 at::Tensor gated_delta_rule(at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor beta_logit, at::Tensor dt,
                             at::Tensor A_log, at::Tensor dt_bias, at::Tensor state, at::Tensor cu, at::Tensor start,
-                            at::Tensor slots, double unit_eps, double q_scale) {
+                            at::Tensor slots, double unit_eps, double q_scale, c10::optional<at::Tensor> chunks,
+                            c10::optional<at::Tensor> seq_chunks) {
   check_rows3(q, "q"); check_rows3(k, "k"); check_rows3(v, "v");
   check_act(beta_logit, "beta_logit"); check_act(dt, "dt");
   const long N = q.size(0);
@@ -392,6 +407,7 @@ at::Tensor gated_delta_rule(at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor
   check_i32(cu, "cu"); check_i32(start, "start"); check_i32(slots, "slots");
   const int B = (int)start.numel();
   const bool head = dt.size(1) == H;
+  const bool chunked = head && chunks.has_value() && seq_chunks.has_value() && D <= DELTA_CHUNK_MAX_D;
   at::Tensor Af = f32c(A_log), bf = f32c(dt_bias);
   TORCH_CHECK(Af.numel() == H && bf.numel() == dt.size(1) && Af.is_cuda() && bf.is_cuda());
   auto fo = q.options().dtype(at::kFloat);
@@ -407,20 +423,17 @@ at::Tensor gated_delta_rule(at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor
                          kn.data_ptr<float>(), decp, beta.data_ptr<float>(), ptr<T>(q),
                          (long)q.stride(0), ptr<T>(k), (long)k.stride(0), ptr<TL>(beta_logit),
                          (long)beta_logit.stride(0), ptr<TL>(dt), (long)dt.stride(0), Af.data_ptr<float>(),
-                         bf.data_ptr<float>(), G, H, D, (float)unit_eps, (float)q_scale);
+                         bf.data_ptr<float>(), G, H, D, (float)unit_eps, (float)q_scale, chunked ? 1 : 0);
     });
     HIP_CHECK_LAST();
-    if (head)
-      launch_scan<SCAN_DELTA_HEAD, T>(out.data_ptr<float>(), qn.data_ptr<float>(), kn.data_ptr<float>(), decp,
-                         beta.data_ptr<float>(), ptr<T>(v), (long)v.stride(0), state.data_ptr<float>(),
-                         (long)state.stride(0), cu.data_ptr<int>(), start.data_ptr<int>(), slots.data_ptr<int>(), B, H,
-                         H / G, D, Dv, (long)G * D, 1, nullptr, N <= 2L * B);
-    else
+    if (!head)
       launch_scan<SCAN_DELTA, T>(out.data_ptr<float>(), qn.data_ptr<float>(), kn.data_ptr<float>(), decp,
                          beta.data_ptr<float>(), ptr<T>(v), (long)v.stride(0), state.data_ptr<float>(),
                          (long)state.stride(0), cu.data_ptr<int>(), start.data_ptr<int>(), slots.data_ptr<int>(), B, H,
                          H / G, D, Dv);
   });
+  if (chunked) delta_head_chunks(out, qn, kn, beta, v.to(at::kFloat), state, start, slots, *chunks, *seq_chunks);
+  else if (head) delta_head_scan(out, qn, kn, beta, v, state, cu, start, slots);
   return out;
 }
 

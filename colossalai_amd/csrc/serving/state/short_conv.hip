@@ -5,7 +5,7 @@
 // the tail refresh (one thread owns all K-1 entries of a (sequence, channel),
 // reads them before it writes), so no element is read and written by
 // different threads of one launch.
-#include "../serving_common.h"
+#include "delta.h"
 
 namespace cai {
 namespace serving {
@@ -62,6 +62,17 @@ __global__ __launch_bounds__(256) void short_conv_tail_kernel(
   }
 }
 
+void refresh_conv_tail(const at::Tensor& x, at::Tensor& tail, const at::Tensor& cu, const at::Tensor& start,
+                       const at::Tensor& slots, int K) {
+  const int C = (int)x.size(1), B = (int)start.numel();
+  SERVING_DISPATCH_ACT(x, T, {
+    hipLaunchKernelGGL(short_conv_tail_kernel<T>, dim3((unsigned)B, (unsigned)((C + 255) / 256)), dim3(256), 0, stream(),
+                       ptr<T>(x), (long)x.stride(0), tail.data_ptr<float>(), (long)tail.stride(0), cu.data_ptr<int>(),
+                       start.data_ptr<int>(), slots.data_ptr<int>(), C, K);
+  });
+  HIP_CHECK_LAST();
+}
+
 at::Tensor short_conv(at::Tensor x, at::Tensor taps, c10::optional<at::Tensor> tail, at::Tensor cu, at::Tensor start,
                       at::Tensor slots, at::Tensor tok_seq, bool silu, at::ScalarType out_dtype,
                       c10::optional<at::Tensor> bias) {
@@ -82,17 +93,14 @@ at::Tensor short_conv(at::Tensor x, at::Tensor taps, c10::optional<at::Tensor> t
   at::Tensor y = at::empty({N, C}, x.options().dtype(out_dtype));
   if (N == 0) return y;
   const float* tlp = nullptr;
-  float* tlw = nullptr;
   long ts = 0;
   if (K > 1) {
     TORCH_CHECK(tail.has_value(), "a convolution with more than one tap carries a tail");
     TORCH_CHECK(is_f32(*tail) && tail->dim() == 3 && tail->size(1) == K - 1 && tail->size(2) == C &&
                 tail->stride(2) == 1 && tail->stride(1) == C, "tail must be float32 [slots, K-1, C]");
-    tlw = tail->data_ptr<float>();
-    tlp = tlw;
+    tlp = tail->data_ptr<float>();
     ts = tail->stride(0);
   }
-  const int B = (int)start.numel();
   const unsigned gy = (unsigned)((C + 255) / 256);
   SERVING_DISPATCH_ACT(x, T, {
     SERVING_DISPATCH_ACT(y, TO, {
@@ -100,12 +108,9 @@ at::Tensor short_conv(at::Tensor x, at::Tensor taps, c10::optional<at::Tensor> t
                          (long)x.stride(0), tp.data_ptr<float>(), tlp, ts, cu.data_ptr<int>(), start.data_ptr<int>(),
                          slots.data_ptr<int>(), tok_seq.data_ptr<int>(), C, K, (int)silu, bp);
     });
-    if (K > 1)
-      hipLaunchKernelGGL(short_conv_tail_kernel<T>, dim3((unsigned)B, gy), dim3(256), 0, stream(), ptr<T>(x),
-                         (long)x.stride(0), tlw, ts, cu.data_ptr<int>(), start.data_ptr<int>(), slots.data_ptr<int>(),
-                         C, K);
   });
   HIP_CHECK_LAST();
+  if (K > 1) refresh_conv_tail(x, *tail, cu, start, slots, K);
   return y;
 }
 

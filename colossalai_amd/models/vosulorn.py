@@ -42,12 +42,11 @@ import torch.nn.functional as F
 
 from ..ops.group_norm import add_rms_norm, grouped_rms_norm, head_rms_norm_gate
 from ..ops.latent_attention import latent_attention, latent_kv_write
-from ..ops.linear_recurrence import gated_delta_rule
+from ..ops.linear_recurrence import conv_gated_delta_rule
 from ..ops.paged_attention import paged_attention
 from ..ops.pair_rotary import halves_to_pairs, pair_frequencies, rotate_qk_write
 from ..ops.ragged import RaggedBatch
 from ..ops.routed_experts import grouped_topk_route, routed_expert_ffn
-from ..ops.short_conv import short_conv
 from .packed import PackedLinear
 from .registry import register_model
 
@@ -203,17 +202,11 @@ class VosulornDelta(nn.Module):
         return buf
 
     def forward(self, h, batch: RaggedBatch, kv, layer: int, state):
-        N = h.shape[0]
         p, y = self.in_proj(h)
-        # the convolution feeds a recurrence: its activated output stays float32
-        qkv = short_conv(y[:, : self.C], self.conv, state.get("tail"), batch, True, torch.float32)
-        q = qkv[:, : self.Cq].view(N, self.G, self.D)
-        k = qkv[:, self.Cq : 2 * self.Cq].view(N, self.G, self.D)
-        v = qkv[:, 2 * self.Cq :].view(N, self.H, self.Dv)
-        o = gated_delta_rule(q, k, v, p["b"], p["a"], self.A_log, self.dt_bias, state["S"], batch, UNIT_EPS,
-                             self.D ** -0.5)
+        o = conv_gated_delta_rule(y[:, : self.C], self.conv, state.get("tail"), self.G, self.D, p["b"], p["a"], self.A_log,
+                                  self.dt_bias, state["S"], batch, UNIT_EPS, self.D ** -0.5)
         o = head_rms_norm_gate(o, self.norm, self.eps, p["g"], h.dtype, act="silu")
-        return self.o(o.view(N, self.Cv))
+        return self.o(o.view(-1, self.Cv))
 
 
 class VosulornMoE(nn.Module):

@@ -21,6 +21,13 @@ Three update rules are provided:
 
 The read-out always includes the current token's write. Gates, decays and the
 state are float32 whatever the activation dtype is.
+
+On the GPU a scan walks a sequence's tokens in order. The delta rule with one
+decay per head has a chunked form besides, taken when a step brings a long
+portion: within 64 tokens the writes solve one triangular system, so everything
+but the state's way from chunk to chunk is float32 matrix products over all
+chunks at once. ``conv_gated_delta_rule`` is that rule with what comes ahead of it
+(short convolution, SiLU, unit length, gates) in one launch.
 """
 
 import torch
@@ -28,9 +35,19 @@ import torch.nn.functional as F
 
 from ._kernels import serving_state_kernels as serving_kernels, use_serving_hip as use_hip
 from .ragged import RaggedBatch
+from .short_conv import short_conv, short_conv_ref
 
-__all__ = ["gated_delta_rule", "gated_delta_rule_ref", "tied_gate_recurrence", "tied_gate_recurrence_ref",
+__all__ = ["gated_delta_rule", "gated_delta_rule_ref", "conv_gated_delta_rule", "conv_gated_delta_rule_ref", "tied_gate_recurrence", "tied_gate_recurrence_ref",
            "ssd_recurrence", "ssd_recurrence_ref"]
+
+
+DELTA_CHUNK = 64          # tokens per chunk (the kernels' own constant)
+DELTA_CHUNKED_FROM = 128  # a step whose longest portion has at least this many tokens runs in chunks
+FUSED_TAPS = 4            # convolution taps the fused inputs kernel takes
+
+
+def _delta_chunks(batch: RaggedBatch):
+    return batch.chunk_tables(DELTA_CHUNK) if batch.max_new >= DELTA_CHUNKED_FROM else (None, None)
 
 
 def _scan_ref(batch, state, n_out, step):
@@ -77,9 +94,40 @@ def gated_delta_rule(q, k, v, beta_logit, dt, A_log, dt_bias, state, batch: Ragg
     channel) or dt [N, H] and dt_bias [H] (one per head); A_log [H];
     state [slots, H, D, Dv] float32. Returns o [N, H, Dv] float32."""
     if use_hip(q):
+        chunks = _delta_chunks(batch) if dt.shape[1] == v.shape[1] else (None, None)
         return serving_kernels().gated_delta_rule(q, k, v, beta_logit, dt, A_log, dt_bias, state, batch.cu,
-                                                  batch.start, batch.slots, unit_eps, q_scale)
+                                                  batch.start, batch.slots, unit_eps, q_scale, *chunks)
     return gated_delta_rule_ref(q, k, v, beta_logit, dt, A_log, dt_bias, state, batch, unit_eps, q_scale)
+
+
+def _after_conv(x, groups: int, dim: int, heads: int):
+    """(q [N, G, D], k [N, G, D], v [N, H, Dv]) views of convolved rows."""
+    N, Cq = x.shape[0], groups * dim
+    return (x[:, :Cq].view(N, groups, dim), x[:, Cq : 2 * Cq].view(N, groups, dim), x[:, 2 * Cq :].view(N, heads, -1))
+
+
+def conv_gated_delta_rule_ref(x, taps, tail, groups: int, dim: int, beta_logit, dt, A_log, dt_bias, state,
+                              batch: RaggedBatch, unit_eps: float = 1e-6, q_scale: float = 1.0):
+    y = short_conv_ref(x, taps, tail, batch, True, torch.float32)
+    return gated_delta_rule_ref(*_after_conv(y, groups, dim, state.shape[1]), beta_logit, dt, A_log, dt_bias, state, batch,
+                                unit_eps, q_scale)
+
+
+def conv_gated_delta_rule(x, taps, tail, groups: int, dim: int, beta_logit, dt, A_log, dt_bias, state,
+                          batch: RaggedBatch, unit_eps: float = 1e-6, q_scale: float = 1.0):
+    """``gated_delta_rule`` with one decay per head, from the projections ahead of the short convolution: x [N, 2 G D +
+    H Dv] (q heads, k heads, v heads; rows may be strided), taps [C, K], tail [slots, K - 1, C] float32 (None for one
+    tap), beta_logit and dt [N, H]. The convolved values stay float32. Returns o [N, H, Dv] float32."""
+    if not use_hip(x):
+        return conv_gated_delta_rule_ref(x, taps, tail, groups, dim, beta_logit, dt, A_log, dt_bias, state, batch, unit_eps,
+                                         q_scale)
+    if taps.shape[1] > FUSED_TAPS:
+        y = short_conv(x, taps, tail, batch, True, torch.float32)
+        return gated_delta_rule(*_after_conv(y, groups, dim, state.shape[1]), beta_logit, dt, A_log, dt_bias, state, batch,
+                                unit_eps, q_scale)
+    return serving_kernels().conv_delta_rule(x, taps, tail, beta_logit, dt, A_log, dt_bias, state, batch.cu, batch.start,
+                                             batch.slots, batch.tok_seq, groups, dim, unit_eps, q_scale,
+                                             *_delta_chunks(batch))
 
 
 def tied_gate_recurrence_ref(q, f_logit, v, f_bias, lower, state, batch: RaggedBatch):

@@ -32,7 +32,7 @@ class RaggedBatch:
     slots_host: List[int]
     page_size: int = 0
     _dense: Optional[dict] = None  # memo of dense_context(), by window
-    _scan_chunks: Optional[tuple] = None  # memo of the selective scan's chunk tables
+    _chunk_tables: Optional[dict] = None  # memo of chunk_tables(), by chunk size
 
     @property
     def num_seqs(self) -> int:
@@ -100,6 +100,23 @@ class RaggedBatch:
             tables = torch.where((cols >= 0) & (cols < pages_d[:, None]), first_d[:, None] + cols, 0).int()
             self._dense[window] = (rows, tables.contiguous(), total)
         return self._dense[window]
+
+    def chunk_tables(self, size: int):
+        """Cut every sequence's new tokens into chunks of ``size``: ``(chunks, seq_chunks)`` with ``chunks`` [K, 4] int32
+        = (sequence, first token, end token, 0) in sequence order and ``seq_chunks`` [B + 1] each sequence's range of
+        chunks, on the device (one copy). Built once per step and size, shared by the step's layers."""
+        if self._chunk_tables is None:
+            self._chunk_tables = {}
+        if size not in self._chunk_tables:
+            rows, ranges = [], [0]
+            for b in range(self.num_seqs):
+                lo, hi = self.cu_host[b], self.cu_host[b + 1]
+                for t in range(lo, hi, size):
+                    rows += [b, t, min(t + size, hi), 0]
+                ranges.append(len(rows) // 4)
+            buf = torch.tensor(rows + ranges, dtype=torch.int32).to(self.cu.device)
+            self._chunk_tables[size] = (buf[: len(rows)].view(-1, 4), buf[len(rows):])
+        return self._chunk_tables[size]
 
     @classmethod
     def build(cls, new_counts: Sequence[int], starts: Sequence[int], slots: Sequence[int], device,

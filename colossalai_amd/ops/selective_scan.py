@@ -34,18 +34,6 @@ CHUNK = 64           # tokens per chunk of the two-pass form (the kernel's own c
 CHUNKED_FROM = 256   # a step whose longest portion has at least this many tokens runs in chunks
 
 
-def _chunk_tables(batch: RaggedBatch):
-    """(chunks [K, 4] int32 = (sequence, first token, end token, 0), seq_chunks [B + 1]) on the device, one copy."""
-    rows, ranges = [], [0]
-    for b in range(batch.num_seqs):
-        lo, hi = batch.cu_host[b], batch.cu_host[b + 1]
-        for t in range(lo, hi, CHUNK):
-            rows += [b, t, min(t + CHUNK, hi), 0]
-        ranges.append(len(rows) // 4)
-    buf = torch.tensor(rows + ranges, dtype=torch.int32).to(batch.cu.device)
-    return buf[: len(rows)].view(-1, 4), buf[len(rows):]
-
-
 def selective_scan_ref(x, dt_raw, A_log, B, C, D_skip, dt_bias, z, state, batch: RaggedBatch, out_dtype=None):
     xf, zf = x.float(), z.float()
     dt = F.softplus(dt_raw.float() + dt_bias.float(), threshold=1e30)      # [N, C], no clamp of large arguments
@@ -69,9 +57,7 @@ def selective_scan(x, dt_raw, A_log, B, C, D_skip, dt_bias, z, state, batch: Rag
     if use_hip(x):
         chunks = seq_chunks = None
         if batch.max_new >= CHUNKED_FROM:
-            if getattr(batch, "_scan_chunks", None) is None:
-                batch._scan_chunks = _chunk_tables(batch)     # once per step, shared by the step's layers
-            chunks, seq_chunks = batch._scan_chunks
+            chunks, seq_chunks = batch.chunk_tables(CHUNK)
         return serving_state_kernels().selective_scan(x, dt_raw, A_log, B, C, D_skip, dt_bias, z, state, batch.cu,
                                                       batch.start, batch.slots, out_dtype or z.dtype, chunks, seq_chunks)
     return selective_scan_ref(x, dt_raw, A_log, B, C, D_skip, dt_bias, z, state, batch, out_dtype)

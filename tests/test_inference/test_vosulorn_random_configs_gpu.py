@@ -86,11 +86,17 @@ def test_random_configuration(seed):
     g = torch.Generator().manual_seed(seed)
     toks = {"a": torch.randint(0, cfg["vocab"], (rng.choice([110, 150]),), generator=g).tolist(),
             "b": torch.randint(0, cfg["vocab"], (rng.choice([3, 40, 70]),), generator=g).tolist()}
-    want = {k: O.forward(cfg, P, v).float() for k, v in toks.items()}
     whole = [[("a", 10 ** 6), ("b", 10 ** 6)]]
     mixed = ([[("a", 37)], [("a", 2), ("b", 5)], [("a", 64), ("b", 1)], [("a", 1), ("b", 30)], [("a", 130), ("b", 1)]]
              + [[("a", 1), ("b", 1)]] * 30 + [[("a", 10 ** 6), ("b", 2)], [("b", 10 ** 6)]])
     for dtype in (torch.float32, torch.bfloat16):
+        if dtype == torch.bfloat16:  # choices that no bfloat16 rounding turns: biases well apart, small products
+            for name in P:
+                if name.endswith("mlp.router"):
+                    P[name] *= 0.1
+                elif name.endswith("mlp.router.b"):
+                    P[name] = torch.linspace(-6, 6, P[name].numel())[torch.randperm(P[name].numel(), generator=g)]
+        want = {k: O.forward(cfg, P, v).float() for k, v in toks.items()}
         for plan in (whole, mixed):
             got = run(cfg, P, toks, dtype, plan)
             err = torch.cat([(got[k] - want[k]).pow(2).mean(-1).sqrt() / want[k].pow(2).mean().sqrt() for k in toks])

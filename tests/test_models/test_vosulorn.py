@@ -18,7 +18,7 @@ from colossalai_amd.models import VosulornForCausalLM, model_class_for  # noqa: 
 from colossalai_amd.models.vosulorn import UNIT_EPS, VosulornMoE  # noqa: E402
 from colossalai_amd.ops import latent_attention as LA  # noqa: E402
 from colossalai_amd.ops.group_norm import head_rms_norm_gate  # noqa: E402
-from colossalai_amd.ops.linear_recurrence import gated_delta_rule  # noqa: E402
+from colossalai_amd.ops.linear_recurrence import conv_gated_delta_rule, gated_delta_rule  # noqa: E402
 from colossalai_amd.ops.paged_attention import paged_attention  # noqa: E402
 from colossalai_amd.ops.pair_rotary import halves_to_pairs, pair_frequencies, rotate_pairs, rotate_qk_write  # noqa: E402
 from colossalai_amd.ops.ragged import RaggedBatch  # noqa: E402
@@ -333,8 +333,9 @@ def test_one_latent_far_back_takes_the_weight(device, far, part):
 
 
 # ------------------------------------------------------------------------- gated delta rule
-def framework_delta(x, taps, b, a, A_log, dt_bias, c, device, cuts, slots=3, slot=1, state=None):
-    """x [T, 2 G D + H Dv] ahead of the convolutions. State buffers start as garbage; returns outputs and final state."""
+def framework_delta(x, taps, b, a, A_log, dt_bias, c, device, cuts, slots=3, slot=1, state=None, fused=True):
+    """x [T, 2 G D + H Dv] ahead of the convolutions. State buffers start as garbage; returns outputs and final state.
+    ``fused``: convolution, unit length and gates through one op, or the convolution and the rule as two."""
     H, G, D, Dv, K = c["heads"], c["kv_heads"], c["dim"], c["vdim"], c["conv"]
     C = x.shape[1]
     if state is None:
@@ -345,12 +346,16 @@ def framework_delta(x, taps, b, a, A_log, dt_bias, c, device, cuts, slots=3, slo
     for n in cuts:
         batch = RaggedBatch.build([n], [at], [slot], device)
         sl = slice(at, at + n)
+        at += n
+        if fused:
+            out.append(conv_gated_delta_rule(x[sl].to(device), taps.to(device), tail, G, D, b[sl].to(device), a[sl].to(device),
+                                             A_log.to(device), dt_bias.to(device), S, batch, UNIT_EPS, D ** -0.5))
+            continue
         y = short_conv(x[sl].to(device), taps.to(device), tail, batch, True, torch.float32)
         Cq = G * D
         out.append(gated_delta_rule(y[:, :Cq].view(n, G, D), y[:, Cq : 2 * Cq].view(n, G, D), y[:, 2 * Cq :].view(n, H, Dv),
                                     b[sl].to(device), a[sl].to(device), A_log.to(device), dt_bias.to(device), S, batch,
                                     UNIT_EPS, D ** -0.5))
-        at += n
     return torch.cat(out, 0), S[slot]
 
 
@@ -383,9 +388,10 @@ def test_delta_rule_in_portions(device, c):
     args = delta_inputs(T, c, 60)
     want, final = oracle_delta(*args)
     for cuts in cuts_of(T, 16) + [[1] * T, [2, 3, 2, 5, 2, 33]]:
-        got, S = framework_delta(*args, device, cuts)
-        close(got, want)
-        close(S, final)
+        for fused in (True, False):
+            got, S = framework_delta(*args, device, cuts, fused=fused)
+            close(got, want)
+            close(S, final)
 
 
 @pytest.mark.parametrize("device", DEVICES)
@@ -398,8 +404,8 @@ def test_delta_rule_over_long_portions(device, c, decay):
     T = 333
     args = delta_inputs(T, c, 70, decay)
     want, final = oracle_delta(*args)
-    for cuts in ([T], [64, 269], [63, 2, 65, 1, 128, 74], [200, 133], [300] + [1] * 33):
-        got, S = framework_delta(*args, device, cuts)
+    for i, cuts in enumerate(([T], [64, 269], [63, 2, 65, 1, 128, 74], [200, 133], [300] + [1] * 33)):
+        got, S = framework_delta(*args, device, cuts, fused=i != 1)
         close(got, want)
         close(S, final)
 
@@ -460,10 +466,8 @@ def test_delta_rule_of_several_sequences(device, lens):
     def step(parts, starts, slots):
         batch = RaggedBatch.build([p[0].shape[0] for p in parts], starts, slots, device)
         x, b, a = (torch.cat([p[i] for p in parts]).to(device) for i in (0, 2, 3))
-        y = short_conv(x, taps.to(device), tail, batch, True, torch.float32)
-        n = x.shape[0]
-        return gated_delta_rule(y[:, :24].view(n, 1, 24), y[:, 24:48].view(n, 1, 24), y[:, 48:].view(n, 3, 16), b, a,
-                                A_log.to(device), dt_bias.to(device), S, batch, UNIT_EPS, 24 ** -0.5)
+        return conv_gated_delta_rule(x, taps.to(device), tail, 1, 24, b, a, A_log.to(device), dt_bias.to(device), S, batch,
+                                     UNIT_EPS, 24 ** -0.5)
 
     slots = [n_slots - 1 - i for i in range(len(lens))]
     cut = lambda s, lo, hi: (s[0][lo:hi], s[1], s[2][lo:hi], s[3][lo:hi])
