@@ -303,7 +303,9 @@ __global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(
 
 // ------------------------------------------------------------------------ chunk scan
 // grid (H, ceil(Dv / 16), B), four waves. Wave w owns tokens 16 w .. 16 w + 15 of a chunk and NT tiles of 16 state rows.
-template <int NT>
+// The loads of the next chunk are issued as soon as this chunk's values have been used, without branches, so that they
+// are in flight over the products in between. VEC: D is a multiple of 4.
+template <int NT, bool VEC>
 __global__ __launch_bounds__(256) void delta_chunk_scan_kernel(
     float* __restrict__ out, ChunkScratch s, const float* __restrict__ q, float* __restrict__ state, long ss,
     const int* __restrict__ start, const int* __restrict__ slots, const int* __restrict__ chunks,
@@ -311,7 +313,7 @@ __global__ __launch_bounds__(256) void delta_chunk_scan_kernel(
   constexpr int Dp = 64 * NT, SP = Dp + 4, UP = CHK + 4, KT = Dp / 16;
   __shared__ __align__(16) float St[16 * SP];   // [column][state row]
   __shared__ __align__(16) float Ut[16 * UP];   // [column][token]
-  const int tid = threadIdx.x, wid = tid >> 6, lane = tid & 63;
+  const int tid = threadIdx.x, wid = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63;
   const int col = lane & 15, g = lane >> 4;
   const int h = blockIdx.x, hq = h / (H / G), slice = blockIdx.y, b = blockIdx.z;
   const int VT = (Dv + 15) >> 4;
@@ -328,7 +330,6 @@ __global__ __launch_bounds__(256) void delta_chunk_scan_kernel(
       const int d = 16 * (wid * NT + j) + 4 * g + r;
       S[j][r] = !fresh && d < D && c < Dv ? Sg[(long)d * Dv + c] : 0.0f;
     }
-  const bool vec = (D & 3) == 0;
   float4v wA[KT], qA[KT], aA[4], kA[NT][4];
   float4v ebr;
   f32x4 uv;
@@ -341,16 +342,13 @@ __global__ __launch_bounds__(256) void delta_chunk_scan_kernel(
 #pragma unroll
     for (int i = 0; i < KT; ++i) {
       wA[i] = *reinterpret_cast<const float4v*>(wr + 16 * i);
-      const int d = 16 * i + 4 * g;
-      float4v val = {0.0f, 0.0f, 0.0f, 0.0f};
-      if (vec) {
-        if (d < D) val = *reinterpret_cast<const float4v*>(qr + d);
+      const int d = 16 * i + 4 * g;   // state rows past D are zero: what they are multiplied with only has to exist
+      if constexpr (VEC) {
+        qA[i] = *reinterpret_cast<const float4v*>(qr + min(d, D - 4));
       } else {
 #pragma unroll
-        for (int e = 0; e < 4; ++e)
-          if (d + e < D) val[e] = qr[d + e];
+        for (int e = 0; e < 4; ++e) qA[i][e] = qr[min(d + e, D - 1)];
       }
-      qA[i] = val;
     }
     uv = *reinterpret_cast<const f32x4*>(s.uv + ((unit * VT + slice) * 4 + wid) * 256 + lane * 4);
   };
@@ -358,8 +356,7 @@ __global__ __launch_bounds__(256) void delta_chunk_scan_kernel(
     const long unit = (long)ck * H + h;
 #pragma unroll
     for (int m = 0; m < 4; ++m) {
-      const float4v none = {0.0f, 0.0f, 0.0f, 0.0f};
-      aA[m] = m <= wid ? *reinterpret_cast<const float4v*>(s.amat + unit * CHK * CHK + (16 * wid + col) * CHK + 16 * m + 4 * g) : none;
+      aA[m] = *reinterpret_cast<const float4v*>(s.amat + unit * CHK * CHK + (16 * wid + col) * CHK + 16 * min(m, wid) + 4 * g);
 #pragma unroll
       for (int j = 0; j < NT; ++j)
         kA[j][m] = *reinterpret_cast<const float4v*>(s.kdt + (unit * Dp + 16 * (wid * NT + j) + col) * CHK + 16 * m + 4 * g);
@@ -387,7 +384,7 @@ __global__ __launch_bounds__(256) void delta_chunk_scan_kernel(
       }
     }
     *reinterpret_cast<f32x4*>(Ut + col * UP + 16 * wid + 4 * g) = u;
-    if (ck + 1 < k1) load_state_side(ck + 1);
+    load_state_side(min(ck + 1, k1 - 1));
     __syncthreads();
 #pragma unroll
     for (int r = 0; r < 4; ++r) oa[r] *= ebr[r];
@@ -402,10 +399,10 @@ __global__ __launch_bounds__(256) void delta_chunk_scan_kernel(
       for (int e = 0; e < 4; ++e) {
 #pragma unroll
         for (int j = 0; j < NT; ++j) S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(kA[j][m][e], ub[e], S[j], 0, 0, 0);
-        oa = __builtin_amdgcn_mfma_f32_16x16x4f32(aA[m][e], ub[e], oa, 0, 0, 0);
       }
+      if (m <= wid) oa = mfma4(aA[m], ub, oa);
     }
-    if (ck + 1 < k1) load_token_side(ck + 1);
+    load_token_side(min(ck + 1, k1 - 1));
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int t = 16 * wid + 4 * g + r;
@@ -443,7 +440,8 @@ static void launch_chunks(at::Tensor& out, const at::Tensor& q, const at::Tensor
   hipLaunchKernelGGL(prep, dim3((unsigned)chunks.size(0), (unsigned)H), dim3(256), smem, stream(), s, q.data_ptr<float>(),
                      k.data_ptr<float>(), gates.data_ptr<float>(), v.data_ptr<float>(), (long)v.stride(0),
                      chunks.data_ptr<int>(), H, G, D, Dv);
-  hipLaunchKernelGGL(delta_chunk_scan_kernel<NT>, dim3((unsigned)H, (unsigned)VT, (unsigned)B), dim3(256), 0, stream(),
+  auto scan = D % 4 == 0 ? delta_chunk_scan_kernel<NT, true> : delta_chunk_scan_kernel<NT, false>;
+  hipLaunchKernelGGL(scan, dim3((unsigned)H, (unsigned)VT, (unsigned)B), dim3(256), 0, stream(),
                      out.data_ptr<float>(), s, q.data_ptr<float>(), state.data_ptr<float>(), (long)state.stride(0),
                      start.data_ptr<int>(), slots.data_ptr<int>(), chunks.data_ptr<int>(), seq_chunks.data_ptr<int>(), H, G,
                      D, Dv);
