@@ -7,7 +7,7 @@
 //                        down products of a token summed with its base row) — only the
 //                        chosen experts' weights are streamed, nothing goes to the host;
 //   expert_sort        : stable counting sort of a step's (token, expert) pairs by expert,
-//                        one block, for the grouped matrix-core product (expert_gemm.hip);
+//                        for the grouped matrix-core product (expert_gemm.hip);
 //   expert_combine     : base + weighted sum of each token's rows of a sorted-by-expert
 //                        output.
 #include "serving_common.h"
@@ -453,7 +453,7 @@ at::Tensor expert_combine(at::Tensor y, at::Tensor inv, at::Tensor weights, c10:
 //   offsets[e] .. offsets[e + 1] = sorted rows of expert e; src[r] = token of sorted row r; inv[p] = sorted row of
 //   pair p. Each wave takes every nw-th expert and walks the pairs 64 at a time (ballot + prefix count), so rows of
 //   one expert keep the order of their pairs and the result does not depend on timing.
-constexpr int SORT_MAX_PAIRS = 8192;
+constexpr int SORT_MAX_PAIRS = 8192;   // of the one-block form
 
 __global__ __launch_bounds__(1024) void expert_sort_kernel(
     int* __restrict__ offsets, int* __restrict__ src, int* __restrict__ inv, const int* __restrict__ ids, int P, int E,
@@ -501,12 +501,81 @@ __global__ __launch_bounds__(1024) void expert_sort_kernel(
   }
 }
 
+// Steps with more pairs: the same order in three launches over tiles of SORT_TILE pairs — counts per (tile, expert),
+// their first sorted rows, then every tile places its pairs.
+constexpr int SORT_TILE = 4096;
+
+__global__ __launch_bounds__(1024) void expert_tile_count_kernel(int* __restrict__ counts, const int* __restrict__ ids,
+                                                                 int P, int E) {
+  __shared__ int held[SORT_TILE];
+  const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63, nw = blockDim.x >> 6;
+  const int base = blockIdx.x * SORT_TILE, cnt = min(SORT_TILE, P - base);
+  for (int p = threadIdx.x; p < cnt; p += blockDim.x) held[p] = ids[base + p];
+  __syncthreads();
+  for (int e = wid; e < E; e += nw) {
+    int n = 0;
+    for (int p0 = 0; p0 < cnt; p0 += 64) n += __popcll(__ballot(p0 + lane < cnt && held[p0 + lane] == e));
+    if (lane == 0) counts[(long)blockIdx.x * E + e] = n;
+  }
+}
+
+// One block, a thread per expert (E <= 1024): counts [tiles, E] become each tile's first row per expert, in place.
+__global__ __launch_bounds__(1024) void expert_tile_offsets_kernel(int* __restrict__ offsets, int* __restrict__ counts,
+                                                                   int tiles, int E) {
+  __shared__ int total[1024];
+  const int e = threadIdx.x;
+  int n = 0;
+  if (e < E)
+    for (int t = 0; t < tiles; ++t) n += counts[(long)t * E + e];
+  total[e] = n;
+  __syncthreads();
+  for (int off = 1; off < 1024; off <<= 1) {   // inclusive running sum over the experts
+    const int up = e >= off ? total[e - off] : 0;
+    __syncthreads();
+    total[e] += up;
+    __syncthreads();
+  }
+  if (e >= E) return;
+  int run = total[e] - n;
+  offsets[e] = run;
+  if (e == E - 1) offsets[E] = total[e];
+  for (int t = 0; t < tiles; ++t) {
+    const int c = counts[(long)t * E + e];
+    counts[(long)t * E + e] = run;
+    run += c;
+  }
+}
+
+__global__ __launch_bounds__(1024) void expert_tile_place_kernel(int* __restrict__ src, int* __restrict__ inv,
+                                                                 const int* __restrict__ firsts,
+                                                                 const int* __restrict__ ids, int P, int E, int top) {
+  __shared__ int held[SORT_TILE];
+  const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63, nw = blockDim.x >> 6;
+  const int base = blockIdx.x * SORT_TILE, cnt = min(SORT_TILE, P - base);
+  for (int p = threadIdx.x; p < cnt; p += blockDim.x) held[p] = ids[base + p];
+  __syncthreads();
+  for (int e = wid; e < E; e += nw) {
+    int at = firsts[(long)blockIdx.x * E + e];
+    for (int p0 = 0; p0 < cnt; p0 += 64) {
+      const int p = p0 + lane;
+      const bool hit = p < cnt && held[p] == e;
+      const unsigned long long mask = __ballot(hit);
+      if (hit) {
+        const int r = at + __popcll(mask & ((1ull << lane) - 1ull));
+        src[r] = (base + p) / top;
+        inv[base + p] = r;
+      }
+      at += __popcll(mask);
+    }
+  }
+}
+
 std::vector<at::Tensor> expert_sort(at::Tensor ids, int64_t num_experts) {
   check_i32(ids, "ids");
   TORCH_CHECK(ids.dim() == 2, "ids must be [N, top]");
+  TORCH_CHECK(ids.numel() < (1L << 30), "too many pairs");
   const int P = (int)ids.numel(), top = (int)ids.size(1), E = (int)num_experts;
-  TORCH_CHECK(P <= SORT_MAX_PAIRS, "too many pairs for the one-block sort");
-  TORCH_CHECK(E >= 1 && (size_t)(P + E + 1) * sizeof(int) <= 64 * 1024);
+  TORCH_CHECK(E >= 1 && E <= 1024, "the sort tells apart 1 to 1024 experts");
   at::Tensor offsets = at::empty({E + 1}, ids.options());
   at::Tensor src = at::empty({P}, ids.options());
   at::Tensor inv = at::empty({ids.size(0), ids.size(1)}, ids.options());
@@ -515,8 +584,19 @@ std::vector<at::Tensor> expert_sort(at::Tensor ids, int64_t num_experts) {
     return {offsets, src, inv};
   }
   // an id outside [0, E) would leave rows of src / inv unwritten: the router never produces one
-  hipLaunchKernelGGL(expert_sort_kernel, dim3(1), dim3(1024), (size_t)(P + E + 1) * sizeof(int), stream(),
-                     offsets.data_ptr<int>(), src.data_ptr<int>(), inv.data_ptr<int>(), ids.data_ptr<int>(), P, E, top);
+  if (P <= SORT_MAX_PAIRS) {
+    hipLaunchKernelGGL(expert_sort_kernel, dim3(1), dim3(1024), (size_t)(P + E + 1) * sizeof(int), stream(),
+                       offsets.data_ptr<int>(), src.data_ptr<int>(), inv.data_ptr<int>(), ids.data_ptr<int>(), P, E, top);
+  } else {
+    const int tiles = (P + SORT_TILE - 1) / SORT_TILE;
+    at::Tensor counts = at::empty({tiles, E}, ids.options());
+    hipLaunchKernelGGL(expert_tile_count_kernel, dim3((unsigned)tiles), dim3(1024), 0, stream(), counts.data_ptr<int>(),
+                       ids.data_ptr<int>(), P, E);
+    hipLaunchKernelGGL(expert_tile_offsets_kernel, dim3(1), dim3(1024), 0, stream(), offsets.data_ptr<int>(),
+                       counts.data_ptr<int>(), tiles, E);
+    hipLaunchKernelGGL(expert_tile_place_kernel, dim3((unsigned)tiles), dim3(1024), 0, stream(), src.data_ptr<int>(),
+                       inv.data_ptr<int>(), counts.data_ptr<int>(), ids.data_ptr<int>(), P, E, top);
+  }
   HIP_CHECK_LAST();
   return {offsets, src, inv};
 }

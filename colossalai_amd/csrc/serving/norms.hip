@@ -116,6 +116,36 @@ __global__ __launch_bounds__(256) void head_rms_norm_gate_kernel(
   }
 }
 
+// The same with eight channels per lane and 1 << lane_shift lanes per (n, h), several of which share a wave (sizes and
+// strides multiples of 8, rows aligned, D <= 512).
+template <typename TI, typename TG, typename TO>
+__global__ __launch_bounds__(256) void head_rms_norm_gate_vec_kernel(
+    TO* __restrict__ out, const TI* __restrict__ x, long xs, const float* __restrict__ w, const TG* __restrict__ gate,
+    long gs, long units, int H, int D, float eps, int silu, int lane_shift) {
+  const int L = 1 << lane_shift, c = 8 * (threadIdx.x & (L - 1));
+  const long unit = ((long)blockIdx.x * blockDim.x + threadIdx.x) >> lane_shift;
+  const bool live = unit < units && c < D;
+  const long u = unit < units ? unit : units - 1;
+  const long n = u / H;
+  const int h = (int)(u % H), cc = live ? c : 0;
+  float v[8], g[8];
+  load8(x + n * xs + (long)h * D + cc, v);
+  if (gate != nullptr) load8(gate + n * gs + (long)h * D + cc, g);
+  float ssq = 0.0f;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) ssq += v[e] * v[e];
+  if (!live) ssq = 0.0f;
+  for (int off = 1; off < L; off <<= 1) ssq += __shfl_xor(ssq, off);
+  const float inv = 1.0f / sqrtf(ssq / (float)D + eps);
+  if (!live) return;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    v[e] *= inv * w[c + e];
+    if (gate != nullptr) v[e] *= silu ? g[e] * sigmoidf_(g[e]) : sigmoidf_(g[e]);
+  }
+  store8(out + u * D + c, v);
+}
+
 at::Tensor head_rms_norm_gate(at::Tensor x, at::Tensor weight, double eps, c10::optional<at::Tensor> gate,
                               at::ScalarType out_dtype, int64_t gate_act) {
   TORCH_CHECK(gate_act == 0 || gate_act == 1, "gate activation: 0 = sigmoid, 1 = silu");
@@ -135,9 +165,25 @@ at::Tensor head_rms_norm_gate(at::Tensor x, at::Tensor weight, double eps, c10::
   }
   const long units = N * H;
   const unsigned grid = (unsigned)((units + 3) / 4);
+  auto al32 = [](const at::Tensor& t) { return reinterpret_cast<uintptr_t>(t.data_ptr()) % (8 * t.element_size()) == 0; };
+  const bool vec = D % 8 == 0 && D <= 512 && x.stride(0) % 8 == 0 && gs % 8 == 0 && al32(x) && al32(out) &&
+                   (!gate.has_value() || al32(*gate));
+  int lane_shift = 0;
+  while ((8 << lane_shift) < D) ++lane_shift;
+  const unsigned vgrid = (unsigned)(((units << lane_shift) + 255) / 256);
   SERVING_DISPATCH_ACT(x, TI, {
     SERVING_DISPATCH_ACT(out, TO, {
-      if (gate.has_value()) {
+      if (vec && gate.has_value()) {
+        SERVING_DISPATCH_ACT(*gate, TG, {
+          hipLaunchKernelGGL((head_rms_norm_gate_vec_kernel<TI, TG, TO>), dim3(vgrid), dim3(256), 0, stream(), ptr<TO>(out),
+                             ptr<TI>(x), (long)x.stride(0), w.data_ptr<float>(), ptr<TG>(*gate), gs, units, H, D,
+                             (float)eps, (int)gate_act, lane_shift);
+        });
+      } else if (vec) {
+        hipLaunchKernelGGL((head_rms_norm_gate_vec_kernel<TI, float, TO>), dim3(vgrid), dim3(256), 0, stream(), ptr<TO>(out),
+                           ptr<TI>(x), (long)x.stride(0), w.data_ptr<float>(), (const float*)nullptr, 0L, units, H, D,
+                           (float)eps, 0, lane_shift);
+      } else if (gate.has_value()) {
         SERVING_DISPATCH_ACT(*gate, TG, {
           hipLaunchKernelGGL((head_rms_norm_gate_kernel<TI, TG, TO>), dim3(grid), dim3(256), 0, stream(), ptr<TO>(out),
                              ptr<TI>(x), (long)x.stride(0), w.data_ptr<float>(), ptr<TG>(*gate), gs, units, H, D,

@@ -133,20 +133,20 @@ def _sort_pairs(ids, E: int):
     return order, inv, offsets
 
 
-SORT_KERNEL_MAX_PAIRS = 8192  # the one-block sort kernel holds a step's ids in LDS
+SORT_KERNEL_MAX_IDS = 1024  # ids the sort kernels tell apart
 
 
 def _grouped_expert_ffn(h, w_up, w_down, ids, weights, base, base_gate=None, activation="relu_squared", sorted_as=None):
     """One grouped matrix-core launch per product; the up product gathers the tokens' rows itself and squares the
-    rectified accumulator (a gated activation runs on the packed product instead). Steps of up to 8192 pairs are
-    sorted by one kernel, larger ones by library sorts. ``sorted_as`` = number of ids the sort tells apart when
+    rectified accumulator (a gated activation runs on the packed product instead). The pairs are sorted by the sort
+    kernels (by library sorts where there are too many ids for them). ``sorted_as`` = number of ids the sort tells apart when
     identity experts follow the real ones: their pairs sort behind every expert's rows, no product touches them and
     the combine step adds ``weight * h`` for them."""
     N, top = ids.shape
     K = serving_kernels()
     E = w_up.shape[0]
     n_ids = sorted_as or E
-    if ids.numel() <= SORT_KERNEL_MAX_PAIRS:
+    if n_ids <= SORT_KERNEL_MAX_IDS:
         offsets, src, inv = K.expert_sort(ids.contiguous(), n_ids)
     else:
         order, inv, offsets = _sort_pairs(ids, n_ids)

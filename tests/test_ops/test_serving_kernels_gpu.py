@@ -372,7 +372,8 @@ def test_expert_grouped_gemm(M, K):
         torch.testing.assert_close(out.cpu().float(), ref, rtol=2e-2, atol=2e-2)
 
 
-@pytest.mark.parametrize("N,top,E", [(1, 1, 1), (40, 3, 7), (1000, 6, 32), (2048, 4, 200), (77, 1, 3)])
+@pytest.mark.parametrize("N,top,E", [(1, 1, 1), (40, 3, 7), (1000, 6, 32), (2048, 4, 200), (77, 1, 3), (4096, 6, 32),
+                                     (3000, 3, 1024), (8193, 1, 5), (12289, 2, 1)])
 def test_expert_sort(N, top, E):
     from colossalai_amd.ops._kernels import serving_kernels
 

@@ -126,10 +126,11 @@ def test_rotation_and_page_write(dtype, shape, H, G, D, Dv, dims, pad):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("N,H,D", [(50, 16, 128), (7, 3, 20), (1, 1, 300)])
-def test_output_norm_with_silu_gate(dtype, N, H, D):
+@pytest.mark.parametrize("N,H,D", [(50, 16, 128), (7, 3, 20), (1, 1, 300), (33, 2, 72), (5, 3, 512), (9, 1, 8)])
+@pytest.mark.parametrize("pad", [8, 3])
+def test_output_norm_with_silu_gate(dtype, N, H, D, pad):
     torch.manual_seed(N)
-    x, w, g = torch.randn(N, H, D), torch.rand(D) + 0.5, torch.randn(N, H * D + 3).to(dtype)
+    x, w, g = torch.randn(N, H, D), torch.rand(D) + 0.5, torch.randn(N, H * D + pad).to(dtype)
     got = head_rms_norm_gate(x.cuda(), w.cuda(), 1e-5, g.cuda()[:, : H * D], dtype, act="silu")
     torch.testing.assert_close(got.cpu(), head_rms_norm_gate_ref(x, w, 1e-5, g[:, : H * D], dtype, act="silu"), **tol(dtype))
 
