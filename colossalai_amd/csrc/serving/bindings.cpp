@@ -54,7 +54,7 @@ at::Tensor query_norm_key_write(at::Tensor q, at::Tensor k, at::Tensor weight, d
                                 at::Tensor positions, at::Tensor kpool, at::Tensor kfac, at::Tensor rows);
 at::Tensor difference_norm(at::Tensor o, int64_t kv_heads, double lam, double mult, double eps, at::ScalarType out_dtype);
 std::vector<at::Tensor> streams_start(at::Tensor table, at::Tensor tokens, int64_t streams, at::Tensor w_in,
-                                      at::Tensor weight, double eps);
+                                      at::Tensor weight, double eps, double scale);
 c10::optional<at::Tensor> streams_update(at::Tensor x, at::Tensor y, at::Tensor mix, at::Tensor w_out,
                                          c10::optional<at::Tensor> w_in, c10::optional<at::Tensor> weight, double eps,
                                          at::ScalarType out_dtype);

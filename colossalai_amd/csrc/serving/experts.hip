@@ -503,7 +503,7 @@ __global__ __launch_bounds__(1024) void expert_sort_kernel(
 
 // Steps with more pairs: the same order in three launches over tiles of SORT_TILE pairs — counts per (tile, expert),
 // their first sorted rows, then every tile places its pairs.
-constexpr int SORT_TILE = 4096;
+constexpr int SORT_TILE = 1024;
 
 __global__ __launch_bounds__(1024) void expert_tile_count_kernel(int* __restrict__ counts, const int* __restrict__ ids,
                                                                  int P, int E) {

@@ -1,7 +1,7 @@
 // Parallel residual streams ("hyper-connections"): instead of one residual row a token carries S rows
 // x_1 .. x_S (float32). A sublayer reads u = sum_s in[s] x_s and, from its output y,
 // x_t <- sum_s mix[s, t] x_s + out[t] y for all t at once from the old rows.
-//   streams_start  : the embedding row becomes every stream, and the first sublayer's input
+//   streams_start  : the (scaled) embedding row becomes every stream, and the first sublayer's input
 //                    rms_norm(u) * w is formed in the same launch;
 //   streams_update : the write of one sublayer, in place, and the read + norm of the next one
 //                    (or of the output, with in = 1 everywhere) in one pass over the streams.
@@ -193,7 +193,7 @@ template <typename TE, int V>
 __global__ __launch_bounds__(256) void streams_start_kernel(TE* __restrict__ h, float* __restrict__ x,
                                                             const TE* __restrict__ table, const long* __restrict__ tokens,
                                                             const float* __restrict__ w_in, const float* __restrict__ w,
-                                                            int W, int S, float eps) {
+                                                            int W, int S, float eps, float scale) {
   __shared__ float red[8];
   const long row = blockIdx.x;
   const TE* er = table + tokens[row] * (long)W;
@@ -206,7 +206,10 @@ __global__ __launch_bounds__(256) void streams_start_kernel(TE* __restrict__ h, 
     if constexpr (V == 4) load4(er + i, e);
     else e[0] = ldf(er + i);
 #pragma unroll
-    for (int k = 0; k < V; ++k) ssq += (total * e[k]) * (total * e[k]);
+    for (int k = 0; k < V; ++k) {
+      e[k] *= scale;
+      ssq += (total * e[k]) * (total * e[k]);
+    }
     for (int s = 0; s < S; ++s) {
       if constexpr (V == 4) store4(xr + (long)s * W + i, e);
       else xr[(long)s * W + i] = e[0];
@@ -221,16 +224,16 @@ __global__ __launch_bounds__(256) void streams_start_kernel(TE* __restrict__ h, 
       load4(er + i, e);
       load4(w + i, wv);
 #pragma unroll
-      for (int k = 0; k < V; ++k) e[k] *= inv * wv[k];
+      for (int k = 0; k < V; ++k) e[k] = e[k] * scale * inv * wv[k];
       store4(h + row * (long)W + i, e);
     } else {
-      stf(h + row * (long)W + i, ldf(er + i) * inv * w[i]);
+      stf(h + row * (long)W + i, ldf(er + i) * scale * inv * w[i]);
     }
   }
 }
 
 std::vector<at::Tensor> streams_start(at::Tensor table, at::Tensor tokens, int64_t streams, at::Tensor w_in,
-                                      at::Tensor weight, double eps) {
+                                      at::Tensor weight, double eps, double scale) {
   check_act(table, "table");
   TORCH_CHECK(table.dim() == 2 && table.is_contiguous(), "table must be contiguous [vocab, W]");
   TORCH_CHECK(tokens.is_cuda() && tokens.scalar_type() == at::kLong && tokens.dim() == 1 && tokens.is_contiguous(),
@@ -248,11 +251,11 @@ std::vector<at::Tensor> streams_start(at::Tensor table, at::Tensor tokens, int64
       if (vec)
         hipLaunchKernelGGL((streams_start_kernel<TE, 4>), dim3((unsigned)N), dim3(256), 0, stream(), ptr<TE>(h),
                            x.data_ptr<float>(), ptr<TE>(table), (const long*)tokens.data_ptr<int64_t>(),
-                           wi.data_ptr<float>(), w.data_ptr<float>(), W, S, (float)eps);
+                           wi.data_ptr<float>(), w.data_ptr<float>(), W, S, (float)eps, (float)scale);
       else
         hipLaunchKernelGGL((streams_start_kernel<TE, 1>), dim3((unsigned)N), dim3(256), 0, stream(), ptr<TE>(h),
                            x.data_ptr<float>(), ptr<TE>(table), (const long*)tokens.data_ptr<int64_t>(),
-                           wi.data_ptr<float>(), w.data_ptr<float>(), W, S, (float)eps);
+                           wi.data_ptr<float>(), w.data_ptr<float>(), W, S, (float)eps, (float)scale);
     });
     HIP_CHECK_LAST();
   }

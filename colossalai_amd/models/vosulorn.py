@@ -40,13 +40,14 @@ import torch
 import torch.nn as nn
 import torch.nn.functional as F
 
-from ..ops.group_norm import add_rms_norm, grouped_rms_norm, head_rms_norm_gate
+from ..ops.group_norm import add_rms_norm, head_rms_norm_gate
 from ..ops.latent_attention import latent_attention, latent_kv_write
 from ..ops.linear_recurrence import conv_gated_delta_rule
 from ..ops.paged_attention import paged_attention
 from ..ops.pair_rotary import halves_to_pairs, pair_frequencies, rotate_qk_write
 from ..ops.ragged import RaggedBatch
 from ..ops.routed_experts import grouped_topk_route, routed_expert_ffn
+from ..ops.streams import streams_start
 from .packed import PackedLinear
 from .registry import register_model
 
@@ -254,11 +255,14 @@ class VosulornForCausalLM(nn.Module):
 
     def __init__(self, cfg: VosulornConfig):
         super().__init__()
+        if not cfg.layers:
+            raise ValueError("a model needs at least one layer")
         self.config = cfg
         self.embed = nn.Embedding(cfg.vocab, cfg.width)
         self.layers = nn.ModuleList([VosulornLayer(cfg, s) for s in cfg.layers])
         self.final_norm = _vec(cfg.width)
         self.head = nn.Linear(cfg.width, cfg.vocab, bias=False)
+        self.register_buffer("one", torch.ones(1), persistent=False)  # the residual as a single stream, read as it is
         for i, layer in enumerate(self.layers):
             a, j = layer.mix, layer.mix.kv_from
             if j is None:
@@ -294,22 +298,24 @@ class VosulornForCausalLM(nn.Module):
         StateCacheManager laid out by ``kv_layer_shapes`` / ``kv_layer_sources`` / ``state_layer_buffers``. Returns
         float32 logits of the rows ``want`` (indices into the flat token axis; all rows if None). ``residuals``, when a
         list, receives a copy of the float32 residual stream after every layer."""
-        cfg, act = self.config, self.act_dtype
-        eps, n = cfg.norm_eps, len(self.layers)
-        x = self.embed(tokens).float() * cfg.embedding_scale
-        h = grouped_rms_norm(x, self.layers[0].norm1, 1, eps, None, act) if n else None
+        cfg, act, n = self.config, self.act_dtype, len(self.layers)
+        eps = cfg.norm_eps
+        x, h = streams_start(self.embed.weight, tokens, 1, self.one, self.layers[0].norm1, eps, cfg.embedding_scale)
+        x = x.view(-1, cfg.width)
         for i, layer in enumerate(self.layers):
-            next_w = self.layers[i + 1].norm1 if i + 1 < n else None
             y = layer.mix(h, batch, kv, i, state.layers[i])
             if layer.mlp is not None:
                 h = add_rms_norm(x, y, None, layer.norm2, eps, act)
                 y = layer.mlp(h)
-            h = add_rms_norm(x, y, None, next_w, eps, act)
+            last = i + 1 == n
+            if last and want is not None and residuals is None:  # the last sum is per row: the wanted rows only
+                x, y = x.index_select(0, want), y.index_select(0, want)
+            h = add_rms_norm(x, y, None, self.final_norm if last else self.layers[i + 1].norm1, eps, act)
             if residuals is not None:
                 residuals.append(x.clone())
-        if want is not None:
-            x = x.index_select(0, want)
-        return self.head(grouped_rms_norm(x, self.final_norm, 1, eps, None, act)).float()
+        if want is not None and residuals is not None:
+            h = h.index_select(0, want)
+        return self.head(h).float()
 
     def forward(self, input_ids: torch.Tensor) -> torch.Tensor:
         """input_ids [B, S] -> logits [B, S, vocab] (float32), every sequence from position 0 with caches that

@@ -6,7 +6,7 @@ formed anew, all at once from the old ones:
 
     x_t <- sum_s mix[s, t] x_s + write[t] * y        (mix indexed [from, to]).
 
-``streams_start`` makes every stream the token's embedding row and forms the first
+``streams_start`` makes every stream the token's (scaled) embedding row and forms the first
 sublayer's normed input. ``streams_update`` does one sublayer's write, in place,
 together with the read and RMS norm of whatever comes next — the next sublayer,
 or the output head, which reads the plain sum (``read=None``) — so each stream
@@ -28,17 +28,17 @@ def _read_norm(x, read, weight, eps, out_dtype):
     return grouped_rms_norm_ref(u, weight, 1, eps, None, out_dtype)
 
 
-def streams_start_ref(table, tokens, streams: int, read, weight, eps: float):
-    x = table[tokens].float()[:, None, :].repeat(1, streams, 1)
+def streams_start_ref(table, tokens, streams: int, read, weight, eps: float, scale: float = 1.0):
+    x = (table[tokens].float() * scale)[:, None, :].repeat(1, streams, 1)
     return x, _read_norm(x, read, weight, eps, table.dtype)
 
 
-def streams_start(table, tokens, streams: int, read, weight, eps: float):
-    """table [vocab, W], tokens [N] int64 -> (streams [N, S, W] float32, ``rms_norm(u) * weight`` in the table's
-    dtype)."""
+def streams_start(table, tokens, streams: int, read, weight, eps: float, scale: float = 1.0):
+    """table [vocab, W], tokens [N] int64 -> (streams [N, S, W] float32 = ``scale`` times the rows, ``rms_norm(u) *
+    weight`` in the table's dtype). With one stream that is the start of an ordinary pre-norm model."""
     if use_hip(table):
-        return tuple(serving_kernels().streams_start(table, tokens, streams, read, weight, eps))
-    return streams_start_ref(table, tokens, streams, read, weight, eps)
+        return tuple(serving_kernels().streams_start(table, tokens, streams, read, weight, eps, float(scale)))
+    return streams_start_ref(table, tokens, streams, read, weight, eps, scale)
 
 
 def streams_update_ref(x, y, mix, write, read, weight, eps: float, out_dtype=None):

@@ -24,6 +24,7 @@ from colossalai_amd.ops.pair_rotary import halves_to_pairs, pair_frequencies, ro
 from colossalai_amd.ops.ragged import RaggedBatch  # noqa: E402
 from colossalai_amd.ops.routed_experts import grouped_topk_route  # noqa: E402
 from colossalai_amd.ops.short_conv import short_conv  # noqa: E402
+from colossalai_amd.ops.streams import streams_start  # noqa: E402
 
 DEVICES = ["cpu", pytest.param("cuda", marks=pytest.mark.gpu)]
 F64 = torch.float64
@@ -520,6 +521,16 @@ def test_expert_layer(device, W, E, top, ff, N):
     with torch.no_grad():
         got = mlp(h.to(device))
     close(got, O.moe(h.to(F64), P, "l0.mlp.", cfg["layers"][0]["mlp"]))
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("W,scale", [(26, 3.5), (64, 1.0), (1030, 0.02)])
+def test_scaled_embedding_and_first_norm(device, W, scale):
+    table, toks, w = rand(150, 11, W), torch.tensor([3, 0, 10, 7, 7]), 1 + 0.3 * rand(151, W)
+    x, h = streams_start(table.to(device), toks.to(device), 1, torch.ones(1, device=device), w.to(device), 1e-4, scale)
+    want = table[toks].to(F64) * scale
+    close(x[:, 0], want, 1e-6)
+    close(h, O.rms_norm(want, w, 1e-4), 1e-5)
 
 
 # -------------------------------------------------------------------- whole models
